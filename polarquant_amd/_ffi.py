@@ -13,7 +13,8 @@ from ctypes import c_char_p, c_float, c_int, c_int64, c_size_t, c_uint, c_void_p
 HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(HERE, "libpolarquant_hip.so")
 
-PQ_F16, PQ_BF16 = 0, 1
+PQ_F16, PQ_BF16, PQ_F32 = 0, 1, 2          # float32: the latent-attention entry points only
+PQ_EPI_PLAIN, PQ_EPI_RELU_SQ, PQ_EPI_SIGMOID_GATE, PQ_EPI_F32 = 0, 1, 2, 3
 PQ_WRAP_FP32 = 1
 PQ_ANGLE_UNIFORM = 2
 PQ_CODES_PACKED6 = 4
@@ -93,53 +94,70 @@ BENCH_SIGNATURES = {
 }
 
 
+# latent attention and the layer steps around it (include/polarquant_latent.h): a library of their own, so that a decoder
+# that needs nothing else need not build the polar-key kernels
+LATENT_LIB_PATH = os.path.join(HERE, "libpolarquant_latent.so")
+LATENT_SIGNATURES = {
+    "pq_norm_conv": (c_int, [c_void_p] * 11 + [c_int] * 6 + [c_float] + [c_int] + [c_void_p]),
+    "pq_validate_norm_conv": (c_int, [c_void_p] * 11 + [c_int] * 7),
+    "pq_latent_norm": (c_int, [c_void_p] + [c_int64] + [c_void_p] * 4 + [c_int64] + [c_void_p] + [c_int] * 5 + [c_float] + [c_int] + [c_void_p]),
+    "pq_validate_latent_norm": (c_int, [c_void_p] + [c_int64] + [c_void_p] * 4 + [c_int64] + [c_void_p] + [c_int] * 6),
+    "pq_relu_sq": (c_int, [c_void_p] * 2 + [c_size_t] + [c_int] + [c_void_p]),
+    "pq_head_linear": (c_int, [c_void_p] + [c_int64] * 2 + [c_void_p] * 2 + [c_int64] + [c_void_p] + [c_int64] * 2 + [c_int] * 6 + [c_void_p]),
+    "pq_validate_head_linear": (c_int, [c_void_p] + [c_int64] * 2 + [c_void_p] * 2 + [c_int64] + [c_void_p] + [c_int64] * 2 + [c_int] * 6),
+    "pq_latent_decode_plan": (c_int, [c_int] * 3 + [c_int64] + [c_int]),
+    "pq_latent_decode_workspace_bytes": (c_size_t, [c_int] * 5),
+    "pq_latent_decode": (c_int, [c_void_p] * 2 + [c_int64] + [c_void_p] * 3 + [c_int] + [c_void_p] + [c_int] * 4 + [c_float] + [c_int] + [c_void_p] + [c_size_t] + [c_int] + [c_void_p]),
+    "pq_validate_latent_decode": (c_int, [c_void_p] * 2 + [c_int64] + [c_void_p] * 3 + [c_int] + [c_void_p] + [c_int] * 5 + [c_void_p] + [c_size_t] + [c_int]),
+    "pq_latent_prefill_takes": (c_int, [c_int] * 3),
+    "pq_latent_prefill": (c_int, [c_void_p] * 3 + [c_int64] + [c_void_p] * 2 + [c_int64] + [c_void_p] * 2 + [c_int] * 6 + [c_float] + [c_int] + [c_void_p]),
+    "pq_validate_latent_prefill": (c_int, [c_void_p] * 3 + [c_int64] + [c_void_p] * 2 + [c_int64] + [c_void_p] * 2 + [c_int] * 7),
+}
+
+
 class PolarQuantError(RuntimeError):
     def __init__(self, status: int, where: str):
         self.status = status
         msg = STATUS_NAMES.get(status, str(status))
         try:
             msg += ": " + lib().pq_status_string(status).decode()
-        except Exception:
+        except Exception:                       # (the polar-key library need not be built)
             pass
         super().__init__("%s failed with %s" % (where, msg))
 
 
-_LIB = None
+_LOADED = {}
+
+
+def _load(path: str, signatures) -> ctypes.CDLL:
+    """The library at `path` with its symbols' types set, loaded once.  Raises if it has not been built."""
+    handle = _LOADED.get(path)
+    if handle is None:
+        if not os.path.exists(path):
+            raise RuntimeError("polarquant_amd: %s is missing; build it with `python -m polarquant_amd.build` "
+                               "(there is no CPU fallback)" % path)
+        handle = ctypes.CDLL(path)
+        for name, (res, args) in signatures.items():
+            fn = getattr(handle, name)
+            fn.restype = res
+            fn.argtypes = args
+        _LOADED[path] = handle
+    return handle
 
 
 def lib() -> ctypes.CDLL:
-    """The loaded HIP library.  Raises if it has not been built."""
-    global _LIB
-    if _LIB is None:
-        if not os.path.exists(LIB_PATH):
-            raise RuntimeError(
-                "polarquant_amd: %s is missing; build it with `python -m polarquant_amd.build` "
-                "(there is no CPU fallback)" % LIB_PATH)
-        handle = ctypes.CDLL(LIB_PATH)
-        for name, (res, args) in SIGNATURES.items():
-            fn = getattr(handle, name)
-            fn.restype = res
-            fn.argtypes = args
-        _LIB = handle
-    return _LIB
+    """The polar-key library."""
+    return _load(LIB_PATH, SIGNATURES)
 
 
-_BENCH_LIB = None
+def latent_lib() -> ctypes.CDLL:
+    """The latent-attention library."""
+    return _load(LATENT_LIB_PATH, LATENT_SIGNATURES)
 
 
 def bench_lib() -> ctypes.CDLL:
-    """The measurement-aid library.  Raises if it has not been built."""
-    global _BENCH_LIB
-    if _BENCH_LIB is None:
-        if not os.path.exists(BENCH_LIB_PATH):
-            raise RuntimeError("polarquant_amd: %s is missing; build it with `python -m polarquant_amd.build`" % BENCH_LIB_PATH)
-        handle = ctypes.CDLL(BENCH_LIB_PATH)
-        for name, (res, args) in BENCH_SIGNATURES.items():
-            fn = getattr(handle, name)
-            fn.restype = res
-            fn.argtypes = args
-        _BENCH_LIB = handle
-    return _BENCH_LIB
+    """The measurement-aid library."""
+    return _load(BENCH_LIB_PATH, BENCH_SIGNATURES)
 
 
 def check(status: int, where: str) -> None:

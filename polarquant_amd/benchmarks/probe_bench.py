@@ -55,9 +55,9 @@ def _direct_bins(args):
     for name, (res, argtypes) in _ffi.SIGNATURES.items():
         fn = getattr(ship, name)
         fn.restype, fn.argtypes = res, argtypes
-    _ffi._LIB = ship
+    _ffi._LOADED[_ffi.LIB_PATH] = ship
     same = quantize_and_pack_nbit(keys[0], sh.rbits, sh.tbits)[0]
-    _ffi._LIB = timed
+    _ffi._LOADED[_ffi.LIB_PATH] = timed
     torch.cuda.synchronize()
     flips = int((outs[0][0] != same).sum())
     print(json.dumps({"library": "shipping" if args.shipping else "probe direct_bins", "config": cfg,

@@ -1,6 +1,7 @@
 """Build recipe of the HIP library: hipcc for gfx950, in-tree.
 
     python -m polarquant_amd.build                    # (re)build polarquant_amd/libpolarquant_hip.so, its test build and libpolarquant_bench.so
+    python -m polarquant_amd.build --latent           # libpolarquant_latent.so alone
     python -m polarquant_amd.build --phase-timers     # the measuring build (benchmarks/phase_timing.py)
     python -m polarquant_amd.build --probe no_values  # a probe build (benchmarks/probe_bench.py)
 
@@ -27,6 +28,9 @@ UNITS = [("pq_attn.hip", ("PQ_DTYPE=0",), ".f16"), ("pq_attn.hip", ("PQ_DTYPE=1"
          ("pq_scores.hip", (), ""), ("pq_quantize.hip", (), ""), ("pq_linear.hip", (), ""), ("pq_attn_common.hip", (), ""),
          ("pq_capi.hip", (), ""), ("pq_values.hip", (), ""), ("pq_decode_ops.hip", (), "")]
 SOURCES = sorted({u[0] for u in UNITS})
+# latent attention and the layer steps around it: a library of their own, all a Dekipel model needs
+LATENT_LIB = os.path.join(HERE, "libpolarquant_latent.so")
+LATENT_UNITS = [("pq_latent.hip", (), ""), ("pq_latent_attn.hip", (), ""), ("pq_head_linear.hip", (), ""), ("pq_latent_capi.hip", (), "")]
 # measurement aids (a plain streaming read, the attention kernel's loads without its arithmetic): a library of
 # their own, loaded by bench.py and its tests only
 BENCH_LIB = os.path.join(HERE, "libpolarquant_bench.so")
@@ -96,6 +100,17 @@ def build_probe(name: str, verbose: bool = True) -> str:
     return PROBE_LIB
 
 
+def build_latent(verbose: bool = True) -> str:
+    """libpolarquant_latent.so alone."""
+    os.makedirs(OBJ, exist_ok=True)
+    with ThreadPoolExecutor(max_workers=len(LATENT_UNITS)) as ex:
+        objs = list(ex.map(lambda j: _compile(*j), LATENT_UNITS))
+    _link(objs, LATENT_LIB)
+    if verbose:
+        print("built", LATENT_LIB)
+    return LATENT_LIB
+
+
 def build(verbose: bool = True, phase_timers: bool = False) -> str:
     """The library the package loads; or, with phase_timers, a second library (same ABI, not loaded by default)
     whose attention kernel times its phases with the wall clock and prints them: a measuring build for
@@ -108,7 +123,7 @@ def build(verbose: bool = True, phase_timers: bool = False) -> str:
         main = list(UNITS)
         hooks = [HOOKS_UNITS.get((src, tag), (src, defs, tag)) for src, defs, tag in UNITS]
         bench = [(s_, (), "") for s_ in BENCH_SOURCES]
-        jobs = main + [u for u in hooks if u not in main] + bench
+        jobs = main + [u for u in hooks if u not in main] + LATENT_UNITS + bench
     # the units are listed longest compilation first
     with ThreadPoolExecutor(max_workers=min(8, len(jobs))) as ex:
         built = dict(zip(jobs, ex.map(lambda j: _compile(*j), jobs)))
@@ -116,8 +131,10 @@ def build(verbose: bool = True, phase_timers: bool = False) -> str:
     _link([built[u] for u in main], lib)
     if not phase_timers:
         _link([built[u] for u in hooks], HOOKS_LIB)
+        _link([built[u] for u in LATENT_UNITS], LATENT_LIB)
         _link([built[u] for u in bench], BENCH_LIB)
         if verbose:
+            print("built", LATENT_LIB)
             print("built", HOOKS_LIB)
             print("built", BENCH_LIB)
     if verbose:
@@ -128,5 +145,7 @@ def build(verbose: bool = True, phase_timers: bool = False) -> str:
 if __name__ == "__main__":
     if "--probe" in sys.argv[1:]:
         build_probe(sys.argv[sys.argv.index("--probe") + 1])
+    elif "--latent" in sys.argv[1:]:
+        build_latent()
     else:
         build(phase_timers="--phase-timers" in sys.argv[1:])

@@ -1,0 +1,374 @@
+// The steps around latent attention: norms, input convolution, projections of small batches.
+//
+//   norm_conv_kernel    residual add of a normed sublayer output, grouped RMS norm of the sum, causal convolution over
+//                       time with its per-sequence state: everything between two sublayers in one launch
+//   latent_norm_kernel  RMS norms of the query latent and of the key/value latent, the latter written to its cache row
+//   relu_sq_kernel      square of relu
+//   head_linear_kernel  per-head (or plain) matrix product for sizes and dtypes the matrix-core kernels do not take
+//
+// All of this is fp32 arithmetic on whatever the operands' dtype is; results are rounded to it once.
+#include "pq_device.h"
+#include "pq_latent_internal.h"
+
+namespace pq {
+
+struct F32 {};
+
+template <typename T> struct Elem { using type = uint16_t; };
+template <> struct Elem<F32> { using type = float; };
+template <typename T> using elem_t = typename Elem<T>::type;
+
+template <typename T> __device__ __forceinline__ float ld1(const elem_t<T>* p) {
+    if constexpr (__is_same(T, F32)) return *p; else return lo2f<T>(*p);
+}
+template <typename T> __device__ __forceinline__ elem_t<T> cv1(float f) {
+    if constexpr (__is_same(T, F32)) return f; else return f2lo<T>(f);
+}
+// V consecutive elements (V 1 or 4; for 4 the address is a multiple of 4 elements)
+template <typename T, int V> __device__ __forceinline__ void ldv(const void* base, size_t i, float (&o)[V]) {
+    const elem_t<T>* p = static_cast<const elem_t<T>*>(base) + i;
+    if constexpr (V == 1) {
+        o[0] = ld1<T>(p);
+    } else if constexpr (__is_same(T, F32)) {
+        const float4 v = *reinterpret_cast<const float4*>(p);
+        o[0] = v.x; o[1] = v.y; o[2] = v.z; o[3] = v.w;
+    } else {
+        const uint2 v = *reinterpret_cast<const uint2*>(p);
+        o[0] = lo2f<T>(static_cast<uint16_t>(v.x & 0xffffu)); o[1] = lo2f<T>(static_cast<uint16_t>(v.x >> 16));
+        o[2] = lo2f<T>(static_cast<uint16_t>(v.y & 0xffffu)); o[3] = lo2f<T>(static_cast<uint16_t>(v.y >> 16));
+    }
+}
+template <typename T, int V> __device__ __forceinline__ void stv(void* base, size_t i, const float (&o)[V]) {
+    elem_t<T>* p = static_cast<elem_t<T>*>(base) + i;
+    if constexpr (V == 1) {
+        *p = cv1<T>(o[0]);
+    } else if constexpr (__is_same(T, F32)) {
+        *reinterpret_cast<float4*>(p) = make_float4(o[0], o[1], o[2], o[3]);
+    } else {
+        *reinterpret_cast<uint2*>(p) = make_uint2(static_cast<uint32_t>(f2lo<T>(o[0])) | (static_cast<uint32_t>(f2lo<T>(o[1])) << 16),
+                                                  static_cast<uint32_t>(f2lo<T>(o[2])) | (static_cast<uint32_t>(f2lo<T>(o[3])) << 16));
+    }
+}
+
+__device__ __forceinline__ float wave_sum(float v) {
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
+    return v;
+}
+
+// ---- residual add + grouped norms + causal convolution ----------------------------------------------------------------
+// A workgroup walks a strip of consecutive tokens of one sequence; a thread owns the same NC pieces of V channels for all
+// of them, so that the last taps - 1 norms (the convolution's inputs) stay in its registers.  A strip that does not begin
+// the call recomputes the norms of the taps - 1 tokens before it (from x_in and y, which nobody overwrites in a call of
+// several strips); the first strip takes them from the state.  TAPS is the register depth: shorter filters are padded
+// with zero taps in front.
+//
+// Sums over a group: where every wavefront's piece lies in one group (`wave_groups`), wavefront sums go through LDS once;
+// otherwise every piece's sum does, and wavefronts add them up group by group.
+template <typename T, int TAPS, int V, int NC>
+__global__ __launch_bounds__(1024) void norm_conv_kernel(NormConvArgs a) {
+    extern __shared__ float lds[];
+    const int tid = threadIdx.x, nthr = blockDim.x, nw = nthr / kWave, wv = tid / kWave, lane = tid & (kWave - 1);
+    const int b = blockIdx.y, W = a.W, L = a.L, taps = a.taps;
+    const int t0 = blockIdx.x * a.strip, t1 = t0 + a.strip < L ? t0 + a.strip : L;
+    const int gs = W / a.groups, pieces = W / V, ppg = gs / V;       // pieces, pieces per group
+    const bool wave_groups = a.groups == 1 || (ppg % kWave) == 0;
+    const int spg = a.groups == 1 ? NC * nw : ppg / kWave;           // wavefront slots per group
+    const float inv_gs = 1.0f / static_cast<float>(gs);
+    const size_t row0 = static_cast<size_t>(b) * L;
+    int phase = 0;
+
+    bool own[NC];
+    int ch[NC];
+#pragma unroll
+    for (int k = 0; k < NC; k++) {
+        const int q = k * nthr + tid;
+        own[k] = q < pieces;
+        ch[k] = (own[k] ? q : 0) * V;
+    }
+    // 1 / sqrt(mean square of the group + eps) for each of this thread's pieces
+    auto group_scale = [&](const float (&v)[NC][V], float (&r)[NC]) {
+        float s[NC];
+#pragma unroll
+        for (int k = 0; k < NC; k++) {
+            s[k] = 0.0f;
+#pragma unroll
+            for (int i = 0; i < V; i++) s[k] = __builtin_fmaf(v[k][i], v[k][i], s[k]);
+            if (!own[k]) s[k] = 0.0f;
+        }
+        if (wave_groups) {
+            float* buf = lds + (phase & 1) * (NC * nw);
+            phase++;
+#pragma unroll
+            for (int k = 0; k < NC; k++) {
+                const float ws = wave_sum(s[k]);
+                if (lane == 0) buf[k * nw + wv] = ws;
+            }
+            __syncthreads();
+#pragma unroll
+            for (int k = 0; k < NC; k++) {
+                const int slot = k * nw + wv, first = (slot / spg) * spg;
+                float sum = 0.0f;
+                for (int j = 0; j < spg; j++) sum += buf[first + j < NC * nw ? first + j : 0];
+                r[k] = rsqrtf(sum * inv_gs + a.eps);
+            }
+        } else {
+            float* buf = lds;
+            float* rs = lds + NC * nthr;
+#pragma unroll
+            for (int k = 0; k < NC; k++) buf[k * nthr + tid] = s[k];
+            __syncthreads();
+            for (int g = wv; g < a.groups; g += nw) {
+                float sum = 0.0f;
+                for (int j = lane; j < ppg; j += kWave) sum += buf[g * ppg + j];
+                sum = wave_sum(sum);
+                if (lane == 0) rs[g] = rsqrtf(sum * inv_gs + a.eps);
+            }
+            __syncthreads();
+#pragma unroll
+            for (int k = 0; k < NC; k++) r[k] = rs[ch[k] / gs];
+        }
+    };
+
+    float wpre[NC][V], wpost[NC][V];
+    constexpr int RING = TAPS > 1 ? TAPS - 1 : 1;
+    float ring[RING][NC][V], cw[TAPS > 0 ? TAPS : 1][NC][V];
+#pragma unroll
+    for (int k = 0; k < NC; k++) {
+        ldv<T, V>(a.w_pre, ch[k], wpre[k]);
+        if (a.y) ldv<T, V>(a.w_post, ch[k], wpost[k]);
+    }
+    if constexpr (TAPS > 0) {
+        const elem_t<T>* w = static_cast<const elem_t<T>*>(a.conv_w);
+#pragma unroll
+        for (int j = 0; j < TAPS; j++) {
+            const int tap = j - (TAPS - taps);               // of the real filter; negative: padding
+#pragma unroll
+            for (int k = 0; k < NC; k++)
+#pragma unroll
+                for (int i = 0; i < V; i++) cw[j][k][i] = tap >= 0 ? ld1<T>(w + static_cast<size_t>(ch[k] + i) * taps + tap) : 0.0f;
+        }
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; j++) {
+            const int row = j - (TAPS - taps);
+#pragma unroll
+            for (int k = 0; k < NC; k++) {
+                if (t0 == 0 && row >= 0)
+                    ldv<F32, V>(a.state_in, (static_cast<size_t>(b) * (taps - 1) + row) * W + ch[k], ring[j][k]);
+                else
+#pragma unroll
+                    for (int i = 0; i < V; i++) ring[j][k][i] = 0.0f;
+            }
+        }
+    }
+    const int first_tok = a.start ? a.start[b] - (a.pos_dev ? *a.pos_dev : a.pos) : 0;      // tokens before it are padding
+    const int begin = (TAPS > 0 && t0 > 0) ? t0 - (taps - 1) : t0;      // strips are longer than the filter
+
+    float xc[NC][V], yc[NC][V], xn[NC][V], yn[NC][V];
+    auto fetch = [&](int t, float (&x)[NC][V], float (&y)[NC][V]) {
+#pragma unroll
+        for (int k = 0; k < NC; k++) {
+            ldv<F32, V>(a.x_in, (row0 + t) * W + ch[k], x[k]);
+            if (a.y) ldv<T, V>(a.y, (row0 + t) * W + ch[k], y[k]);
+        }
+    };
+    fetch(begin, xc, yc);
+    for (int t = begin; t < t1; t++) {
+        if (t + 1 < t1) fetch(t + 1, xn, yn);
+        if (a.y) {
+            float r[NC];
+            group_scale(yc, r);
+#pragma unroll
+            for (int k = 0; k < NC; k++)
+#pragma unroll
+                for (int i = 0; i < V; i++) xc[k][i] += wpost[k][i] * (yc[k][i] * r[k]);
+            if (t >= t0 && a.x_out)
+#pragma unroll
+                for (int k = 0; k < NC; k++)
+                    if (own[k]) stv<F32, V>(a.x_out, (row0 + t) * W + ch[k], xc[k]);
+        }
+        float r[NC];
+        group_scale(xc, r);
+        const bool real = t >= first_tok;
+#pragma unroll
+        for (int k = 0; k < NC; k++) {
+            float h[V], o[V];
+#pragma unroll
+            for (int i = 0; i < V; i++) {
+                h[i] = real ? wpre[k][i] * (xc[k][i] * r[k]) : 0.0f;
+                o[i] = h[i];
+            }
+            if constexpr (TAPS > 0) {
+#pragma unroll
+                for (int i = 0; i < V; i++) {
+                    float c = cw[TAPS - 1][k][i] * h[i];
+#pragma unroll
+                    for (int j = 0; j < TAPS - 1; j++) c = __builtin_fmaf(cw[j][k][i], ring[j][k][i], c);
+                    if (real) o[i] += c;
+#pragma unroll
+                    for (int j = 0; j + 1 < TAPS - 1; j++) ring[j][k][i] = ring[j + 1][k][i];
+                    if constexpr (TAPS > 1) ring[TAPS > 1 ? TAPS - 2 : 0][k][i] = h[i];
+                }
+            }
+            if (t >= t0 && own[k]) stv<T, V>(a.h_out, (row0 + t) * W + ch[k], o);
+        }
+#pragma unroll
+        for (int k = 0; k < NC; k++)
+#pragma unroll
+            for (int i = 0; i < V; i++) { xc[k][i] = xn[k][i]; yc[k][i] = yn[k][i]; }
+    }
+    if constexpr (TAPS > 1) {
+        if (t1 == L) {
+#pragma unroll
+            for (int j = 0; j < TAPS - 1; j++) {
+                const int row = j - (TAPS - taps);
+                if (row < 0) continue;
+#pragma unroll
+                for (int k = 0; k < NC; k++)
+                    if (own[k]) stv<F32, V>(a.state_out, (static_cast<size_t>(b) * (taps - 1) + row) * W + ch[k], ring[j][k]);
+            }
+        }
+    }
+}
+
+int launch_norm_conv(const NormConvArgs& args, int dtype, hipStream_t st) {
+    NormConvArgs a = args;
+    const int taps = a.conv_w ? a.taps : 0;
+    if (!a.conv_w) a.taps = 1;
+    const int V = ((a.W / a.groups) % 4 == 0) ? 4 : 1;
+    const int pieces = a.W / V;
+    const int nthr = pieces <= 256 ? 256 : pieces <= 512 ? 512 : 1024;
+    const int per = (pieces + nthr - 1) / nthr;
+    const int NC = per <= 1 ? 1 : per <= 2 ? 2 : 4;
+    if (per > 4) return static_cast<int>(hipErrorInvalidValue);
+    a.strip = a.L <= kConvInPlaceTokens ? a.L : 32;
+    const size_t shared = (static_cast<size_t>(NC) * nthr + a.groups + 2 * NC * (nthr / kWave)) * sizeof(float);
+    if (shared > 64 * 1024) return static_cast<int>(hipErrorInvalidValue);
+    dim3 grid(static_cast<unsigned>((a.L + a.strip - 1) / a.strip), static_cast<unsigned>(a.B)), block(nthr);
+#define PQ_NC(T, TP, VV, N) hipLaunchKernelGGL((norm_conv_kernel<T, TP, VV, N>), grid, block, shared, st, a)
+#define PQ_NC_N(T, TP, VV) do { if (NC == 1) PQ_NC(T, TP, VV, 1); else if (NC == 2) PQ_NC(T, TP, VV, 2); else PQ_NC(T, TP, VV, 4); } while (0)
+#define PQ_NC_V(T, TP) do { if (V == 4) PQ_NC_N(T, TP, 4); else PQ_NC_N(T, TP, 1); } while (0)
+#define PQ_NC_T(T)                                                                                                   \
+    do {                                                                                                             \
+        if (taps == 0) PQ_NC_V(T, 0);                                                                                \
+        else if (taps <= 4) PQ_NC_V(T, 4);                                                                           \
+        else if (taps <= 8) PQ_NC_V(T, 8);                                                                           \
+        else PQ_NC_V(T, 16);                                                                                         \
+    } while (0)
+    if (dtype == 0) PQ_NC_T(F16); else if (dtype == 1) PQ_NC_T(BF16); else PQ_NC_T(F32);
+#undef PQ_NC_T
+#undef PQ_NC_V
+#undef PQ_NC_N
+#undef PQ_NC
+    return static_cast<int>(hipGetLastError());
+}
+
+// ---- norms of the two latents ---------------------------------------------------------------------------------------
+// One workgroup per token.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void latent_norm_kernel(LatentNormArgs a) {
+    __shared__ float part[2][4];
+    const int tok = blockIdx.x, b = tok / a.L, t = tok - b * a.L, tid = threadIdx.x;
+    const int Q = a.q_rank, R = a.w_kv ? a.kv_rank : 0;
+    const size_t in = static_cast<size_t>(tok) * a.row_stride;
+    float sq = 0.0f, sc = 0.0f, v[V];
+    for (int i = tid * V; i < Q + R; i += 256 * V) {
+        ldv<T, V>(a.p, in + i, v);
+        float s = 0.0f;
+#pragma unroll
+        for (int j = 0; j < V; j++) s = __builtin_fmaf(v[j], v[j], s);
+        if (i < Q) sq += s; else sc += s;
+    }
+    sq = wave_sum(sq);
+    sc = wave_sum(sc);
+    if ((tid & 63) == 0) { part[0][tid >> 6] = sq; part[1][tid >> 6] = sc; }
+    __syncthreads();
+    const float rq = rsqrtf((part[0][0] + part[0][1] + part[0][2] + part[0][3]) / static_cast<float>(Q) + a.eps);
+    const float rc = R ? rsqrtf((part[1][0] + part[1][1] + part[1][2] + part[1][3]) / static_cast<float>(R) + a.eps) : 0.0f;
+    int64_t pos = (a.pos_dev ? *a.pos_dev : a.pos) + t;
+    pos = pos < 0 ? 0 : (pos >= a.capacity ? a.capacity - 1 : pos);          // (never past the cache)
+    const size_t qo = static_cast<size_t>(tok) * Q, co = (static_cast<size_t>(b) * a.capacity + pos) * R;
+    for (int i = tid * V; i < Q + R; i += 256 * V) {
+        float w[V];
+        ldv<T, V>(a.p, in + i, v);
+        if (i < Q) ldv<T, V>(a.w_q, i, w); else ldv<T, V>(a.w_kv, i - Q, w);
+        const float r = i < Q ? rq : rc;
+#pragma unroll
+        for (int j = 0; j < V; j++) v[j] = w[j] * (v[j] * r);
+        if (i < Q) stv<T, V>(a.q_out, qo + i, v); else stv<T, V>(a.cache, co + (i - Q), v);
+    }
+}
+
+int launch_latent_norm(const LatentNormArgs& a, int dtype, hipStream_t st) {
+    const bool v4 = a.q_rank % 4 == 0 && a.kv_rank % 4 == 0 && a.row_stride % 4 == 0;
+    dim3 grid(static_cast<unsigned>(a.B * a.L)), block(256);
+#define PQ_LN(T) do { if (v4) hipLaunchKernelGGL((latent_norm_kernel<T, 4>), grid, block, 0, st, a); \
+                      else hipLaunchKernelGGL((latent_norm_kernel<T, 1>), grid, block, 0, st, a); } while (0)
+    if (dtype == 0) PQ_LN(F16); else if (dtype == 1) PQ_LN(BF16); else PQ_LN(F32);
+#undef PQ_LN
+    return static_cast<int>(hipGetLastError());
+}
+
+// ---- square of relu ----------------------------------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void relu_sq_kernel(const void* __restrict__ x, void* __restrict__ y, size_t n) {
+    const size_t i = (static_cast<size_t>(blockIdx.x) * 256 + threadIdx.x) * 8;
+    if (i + 8 <= n) {
+        float v[2][4];
+        ldv<T, 4>(x, i, v[0]);
+        ldv<T, 4>(x, i + 4, v[1]);
+#pragma unroll
+        for (int k = 0; k < 2; k++)
+#pragma unroll
+            for (int j = 0; j < 4; j++) { const float r = fmaxf(v[k][j], 0.0f); v[k][j] = r * r; }
+        stv<T, 4>(y, i, v[0]);
+        stv<T, 4>(y, i + 4, v[1]);
+    } else {
+        for (size_t j = i; j < n; j++) {
+            const float r = fmaxf(ld1<T>(static_cast<const elem_t<T>*>(x) + j), 0.0f);
+            static_cast<elem_t<T>*>(y)[j] = cv1<T>(r * r);
+        }
+    }
+}
+
+int launch_relu_sq(const void* x, void* y, size_t n, int dtype, hipStream_t st) {
+    dim3 grid(static_cast<unsigned>((n + 2047) / 2048)), block(256);
+    if (dtype == 0) hipLaunchKernelGGL(relu_sq_kernel<F16>, grid, block, 0, st, x, y, n);
+    else if (dtype == 1) hipLaunchKernelGGL(relu_sq_kernel<BF16>, grid, block, 0, st, x, y, n);
+    else hipLaunchKernelGGL(relu_sq_kernel<F32>, grid, block, 0, st, x, y, n);
+    return static_cast<int>(hipGetLastError());
+}
+
+// ---- per-head product, any size ------------------------------------------------------------------------------------------
+// A wavefront per output: lanes stride over k, then a butterfly sum.  grid (N / 4 rounded up, heads, M).
+template <typename T>
+__global__ __launch_bounds__(256) void head_linear_kernel(HeadLinearArgs a) {
+    const int lane = threadIdx.x & 63, n = blockIdx.x * 4 + (threadIdx.x >> 6), h = blockIdx.y, m = blockIdx.z;
+    if (n >= a.N) return;
+    const elem_t<T>* x = static_cast<const elem_t<T>*>(a.x) + m * a.x_row + h * a.x_head;
+    const elem_t<T>* w = static_cast<const elem_t<T>*>(a.w) + (static_cast<size_t>(h) * a.N + n) * a.K;
+    float s = 0.0f;
+    for (int k = lane; k < a.K; k += 64) s = __builtin_fmaf(ld1<T>(x + k), ld1<T>(w + k), s);
+    s = wave_sum(s);
+    if (lane != 0) return;
+    if (a.epilogue == kEpiReluSq) {
+        s = fmaxf(s, 0.0f);
+        s = s * s;
+    } else if (a.epilogue == kEpiSigmoidGate) {
+        const float g = ld1<T>(static_cast<const elem_t<T>*>(a.gate) + m * a.gate_row + static_cast<size_t>(h) * a.N + n);
+        s = s / (1.0f + __expf(-g));
+    }
+    const size_t o = m * a.y_row + h * a.y_head + n;
+    if (a.epilogue == kEpiF32) static_cast<float*>(a.y)[o] = s;
+    else static_cast<elem_t<T>*>(a.y)[o] = cv1<T>(s);
+}
+
+int launch_head_linear_any(const HeadLinearArgs& a, int dtype, hipStream_t st) {
+    dim3 grid(static_cast<unsigned>((a.N + 3) / 4), static_cast<unsigned>(a.heads), static_cast<unsigned>(a.M)), block(256);
+    if (dtype == 0) hipLaunchKernelGGL(head_linear_kernel<F16>, grid, block, 0, st, a);
+    else if (dtype == 1) hipLaunchKernelGGL(head_linear_kernel<BF16>, grid, block, 0, st, a);
+    else hipLaunchKernelGGL(head_linear_kernel<F32>, grid, block, 0, st, a);
+    return static_cast<int>(hipGetLastError());
+}
+
+}  // namespace pq

@@ -1,258 +1,9 @@
-// Linear layers of the decode step: y[M, N] = x[M, K] . W[N, K]^T (+ bias) with M <= 16 rows
-// (one new token per sequence), the q/k/v, o and MLP projections around the attention call
-// (models/modeling_llama_polar.py:47-52, :131 and the decoder layer's MLP, :456-486).
-//
-// At M <= 16 the product is a stream of the weight matrix through HBM, 2*M flops per weight
-// byte: the kernels are laid out for the stream, not for the matrix cores.  Two of them:
-// small_m_linear_kernel (any M <= 16, described here) and small_m8_linear_kernel (M <= 8, further
-// down: whole-line loads, half the x operand traffic).  A workgroup owns
-// 16 output columns (16 rows of W) and splits K over its KSPLIT wavefronts; each wavefront
-// keeps two stages of kStage 16-byte loads per lane in flight (ping-pong) and feeds them to
-// v_mfma_f32_16x16x32 with the W rows as the A operand and x (rows >= M unused) as the B operand:
-// lane l holds W[n0 + l % 16][k + 8 * (l / 16) .. + 8) and x[l % 16][same k], so a 16-byte
-// load per lane is one MFMA operand and a wavefront load covers 16 rows x 64 contiguous
-// bytes.  The KSPLIT partial 16x16 tiles are added in a fixed order through LDS, so results
-// do not depend on scheduling.  x (at most 16 x K) is re-read by every workgroup from L2.
-//
-// GATED: two weight matrices share the x operand and the epilogue applies
-// silu(gate) * up with the eager modules' roundings (gate, up and silu(gate) each rounded
-// to the activation dtype), which saves the [M, 2 * N] round trip and one launch.
-#include "pq_device.h"
+// Launchers of the decode step's linear layers (kernels: pq_linear_device.h), and the q|k|v projection with RoPE and the
+// cache appends in its epilogue.
 #include "pq_internal.h"
+#include "pq_linear_device.h"
 
 namespace pq {
-
-typedef float floatx4_l __attribute__((ext_vector_type(4)));
-typedef uint32_t u32x4_l __attribute__((ext_vector_type(4)));
-typedef _Float16 half8_l __attribute__((ext_vector_type(8)));
-typedef __bf16 bf16x8_l __attribute__((ext_vector_type(8)));
-
-template <typename T> __device__ __forceinline__ floatx4_l mfma32(u32x4_l a, u32x4_l b, floatx4_l c);
-template <> __device__ __forceinline__ floatx4_l mfma32<F16>(u32x4_l a, u32x4_l b, floatx4_l c) {
-    return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(half8_l, a), __builtin_bit_cast(half8_l, b), c, 0, 0, 0);
-}
-template <> __device__ __forceinline__ floatx4_l mfma32<BF16>(u32x4_l a, u32x4_l b, floatx4_l c) {
-    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_l, a), __builtin_bit_cast(bf16x8_l, b), c, 0, 0, 0);
-}
-
-template <typename T>
-__device__ __forceinline__ float rnd_l(float f) { return lo2f<T>(f2lo<T>(f)); }
-
-template <bool GATED, int kStage>
-struct StageT {
-    u32x4_l w[kStage], x[kStage], u[GATED ? kStage : 1];
-};
-
-template <typename T, int KSPLIT, bool GATED, int kStage>
-__global__ __launch_bounds__(kWave * KSPLIT) void small_m_linear_kernel(
-    const uint16_t* __restrict__ x, int64_t x_stride, const uint16_t* __restrict__ w, const uint16_t* __restrict__ w_up,
-    const uint16_t* __restrict__ bias, uint16_t* __restrict__ y, int64_t y_stride, int M, int K) {
-    __shared__ float part[KSPLIT][GATED ? 2 : 1][4][kWave];
-    const int lane = threadIdx.x & (kWave - 1), wv = threadIdx.x / kWave;
-    const int r = lane & 15, g = lane >> 4;
-    const int n0 = blockIdx.x * 16;
-    const int klen = K / KSPLIT, steps = klen / 32;
-    const int m = r < M ? r : 0;                           // tile columns >= M repeat row 0 and are never stored
-    const size_t koff = static_cast<size_t>(wv) * klen + 8 * g;
-    const uint16_t* wp = w + static_cast<size_t>(n0 + r) * K + koff;
-    const uint16_t* up = GATED ? w_up + static_cast<size_t>(n0 + r) * K + koff : nullptr;
-    const uint16_t* xp = x + static_cast<size_t>(m) * x_stride + koff;
-
-    floatx4_l acc[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}}, acu[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}};
-    // No branch may sit between a stage's loads and the MFMAs of the other stage: at a join the
-    // compiler has to wait for every outstanding load, which would serialize the two stages.  So
-    // whole stages run in a branch-free ping-pong loop, and only the tail is predicated.
-    auto load = [&](StageT<GATED, kStage>& st, int s0) {
-        static_for<kStage>([&](auto U) {
-            constexpr int u = decltype(U)::value;
-            st.w[u] = *reinterpret_cast<const u32x4_l*>(wp + (s0 + u) * 32);
-            if constexpr (GATED) st.u[u] = *reinterpret_cast<const u32x4_l*>(up + (s0 + u) * 32);
-            st.x[u] = *reinterpret_cast<const u32x4_l*>(xp + (s0 + u) * 32);
-        });
-    };
-    auto compute = [&](const StageT<GATED, kStage>& st) {
-        static_for<kStage>([&](auto U) {
-            constexpr int u = decltype(U)::value;
-            acc[u & 1] = mfma32<T>(st.w[u], st.x[u], acc[u & 1]);
-            if constexpr (GATED) acu[u & 1] = mfma32<T>(st.u[u], st.x[u], acu[u & 1]);
-        });
-    };
-    const int full = steps / kStage;          // whole stages
-    if (full > 0) {
-        StageT<GATED, kStage> sa, sb;
-        load(sa, 0);
-        int st = 0;
-        while (st + 2 < full) {
-            load(sb, (st + 1) * kStage);
-            compute(sa);
-            load(sa, (st + 2) * kStage);
-            compute(sb);
-            st += 2;
-        }
-        if (full - st == 2) {
-            load(sb, (st + 1) * kStage);
-            compute(sa);
-            compute(sb);
-        } else {
-            compute(sa);
-        }
-    }
-    for (int s1 = full * kStage; s1 < steps; s1++) {      // fewer than kStage steps left
-        const u32x4_l wv1 = *reinterpret_cast<const u32x4_l*>(wp + s1 * 32);
-        const u32x4_l xv1 = *reinterpret_cast<const u32x4_l*>(xp + s1 * 32);
-        acc[0] = mfma32<T>(wv1, xv1, acc[0]);
-        if constexpr (GATED) acu[0] = mfma32<T>(*reinterpret_cast<const u32x4_l*>(up + s1 * 32), xv1, acu[0]);
-    }
-#pragma unroll
-    for (int i = 0; i < 4; i++) {
-        part[wv][0][i][lane] = acc[0][i] + acc[1][i];
-        if constexpr (GATED) part[wv][1][i][lane] = acu[0][i] + acu[1][i];
-    }
-    __syncthreads();
-    if (wv != 0 || r >= M) return;
-    // the MFMA result layout: lane (r, g) holds tile rows 4g + i (i < 4) of tile column r = outputs y[r][n0 + 4g + i]
-    uint16_t out[4];
-#pragma unroll
-    for (int i = 0; i < 4; i++) {
-        float s = part[0][0][i][lane];
-#pragma unroll
-        for (int k = 1; k < KSPLIT; k++) s += part[k][0][i][lane];
-        if constexpr (GATED) {
-            float t = part[0][1][i][lane];
-#pragma unroll
-            for (int k = 1; k < KSPLIT; k++) t += part[k][1][i][lane];
-            const float gv = rnd_l<T>(s), uv = rnd_l<T>(t);
-            const float a = rnd_l<T>(gv / (1.0f + __expf(-gv)));
-            out[i] = f2lo<T>(a * uv);
-        } else {
-            if (bias) s += lo2f<T>(bias[n0 + 4 * g + i]);
-            out[i] = f2lo<T>(s);
-        }
-    }
-    *reinterpret_cast<uint2*>(y + static_cast<size_t>(r) * y_stride + n0 + 4 * g) =
-        make_uint2(static_cast<uint32_t>(out[0]) | (static_cast<uint32_t>(out[1]) << 16),
-                   static_cast<uint32_t>(out[2]) | (static_cast<uint32_t>(out[3]) << 16));
-}
-
-// M <= 8: each 16 x 16 MFMA tile is used as two 8 x 8 tiles on its diagonal.  Tile rows 0-7 are 8 rows
-// of W over the first 32 of a 64-wide k-step, tile rows 8-15 the SAME 8 rows over the second 32; tile
-// columns 0-7 are the rows of x over the first 32, columns 8-15 over the second 32.  Then
-// y[m][n] = C[n][m] + C[n + 8][m + 8] and the off-diagonal quarters are ignored.  No lane loads a
-// duplicate row of x, a wavefront load of W covers 8 rows x 128 contiguous bytes (whole cache lines,
-// which is what lets the weight stream carry the non-temporal hint: with half lines the hint drops a
-// line before its second half is asked for), and the workgroup's 16 rows of W are two such tiles that
-// share one x operand: per 64-wide step two W loads and one x load instead of four and four.
-template <bool GATED, int kStage>
-struct Stage8T {
-    u32x4_l w[2][kStage], x[kStage], u[GATED ? 2 : 1][GATED ? kStage : 1];
-};
-
-template <typename T, int KSPLIT, bool GATED, int kStage>
-__global__ __launch_bounds__(kWave * KSPLIT) void small_m8_linear_kernel(
-    const uint16_t* __restrict__ x, int64_t x_stride, const uint16_t* __restrict__ w, const uint16_t* __restrict__ w_up,
-    const uint16_t* __restrict__ bias, uint16_t* __restrict__ y, int64_t y_stride, int M, int K) {
-    __shared__ float part[KSPLIT][GATED ? 4 : 2][4][kWave];
-    const int lane = threadIdx.x & (kWave - 1), wv = threadIdx.x / kWave;
-    const int r = lane & 15, g = lane >> 4;
-    const int row = r & 7, chunk = (r >> 3) * 4 + g;       // W row inside an 8-row tile == x row; 16-byte piece of the step
-    const int n0 = blockIdx.x * 16;
-    const int klen = K / KSPLIT, steps = klen / 64;
-    const int m = row < M ? row : 0;                       // tile columns >= M repeat row 0 and are never stored
-    const size_t koff = static_cast<size_t>(wv) * klen + 8 * chunk;
-    const uint16_t* wp = w + static_cast<size_t>(n0 + row) * K + koff;
-    const uint16_t* up = GATED ? w_up + static_cast<size_t>(n0 + row) * K + koff : nullptr;
-    const uint16_t* xp = x + static_cast<size_t>(m) * x_stride + koff;
-    const size_t half_tile = static_cast<size_t>(8) * K;   // rows n0 + 8 .. n0 + 15
-
-    floatx4_l acc[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}}, acu[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}};
-    auto ldw = [](const uint16_t* p) { return __builtin_nontemporal_load(reinterpret_cast<const u32x4_l*>(p)); };
-    auto load = [&](Stage8T<GATED, kStage>& st, int s0) {          // branch-free, see small_m_linear_kernel
-        static_for<kStage>([&](auto U) {
-            constexpr int u = decltype(U)::value;
-            st.w[0][u] = ldw(wp + (s0 + u) * 64);
-            st.w[1][u] = ldw(wp + half_tile + (s0 + u) * 64);
-            if constexpr (GATED) {
-                st.u[0][u] = ldw(up + (s0 + u) * 64);
-                st.u[1][u] = ldw(up + half_tile + (s0 + u) * 64);
-            }
-            st.x[u] = *reinterpret_cast<const u32x4_l*>(xp + (s0 + u) * 64);
-        });
-    };
-    auto compute = [&](const Stage8T<GATED, kStage>& st) {
-        static_for<kStage>([&](auto U) {
-            constexpr int u = decltype(U)::value;
-            acc[0] = mfma32<T>(st.w[0][u], st.x[u], acc[0]);
-            acc[1] = mfma32<T>(st.w[1][u], st.x[u], acc[1]);
-            if constexpr (GATED) {
-                acu[0] = mfma32<T>(st.u[0][u], st.x[u], acu[0]);
-                acu[1] = mfma32<T>(st.u[1][u], st.x[u], acu[1]);
-            }
-        });
-    };
-    const int full = steps / kStage;
-    if (full > 0) {
-        Stage8T<GATED, kStage> sa, sb;
-        load(sa, 0);
-        int st = 0;
-        while (st + 2 < full) {
-            load(sb, (st + 1) * kStage);
-            compute(sa);
-            load(sa, (st + 2) * kStage);
-            compute(sb);
-            st += 2;
-        }
-        if (full - st == 2) {
-            load(sb, (st + 1) * kStage);
-            compute(sa);
-            compute(sb);
-        } else {
-            compute(sa);
-        }
-    }
-    for (int s1 = full * kStage; s1 < steps; s1++) {
-        const u32x4_l xv1 = *reinterpret_cast<const u32x4_l*>(xp + s1 * 64);
-        acc[0] = mfma32<T>(ldw(wp + s1 * 64), xv1, acc[0]);
-        acc[1] = mfma32<T>(ldw(wp + half_tile + s1 * 64), xv1, acc[1]);
-        if constexpr (GATED) {
-            acu[0] = mfma32<T>(ldw(up + s1 * 64), xv1, acu[0]);
-            acu[1] = mfma32<T>(ldw(up + half_tile + s1 * 64), xv1, acu[1]);
-        }
-    }
-#pragma unroll
-    for (int i = 0; i < 4; i++) {
-        part[wv][0][i][lane] = acc[0][i];
-        part[wv][1][i][lane] = acc[1][i];
-        if constexpr (GATED) { part[wv][2][i][lane] = acu[0][i]; part[wv][3][i][lane] = acu[1][i]; }
-    }
-    __syncthreads();
-    // lane (r < 8, g < 2) owns outputs y[r][n0 + 8h + 4g + i] (h: which 8-row tile), each the sum of the tile's
-    // entry (row 4g + i, column r) and its diagonal partner (row + 8, column + 8), which lane + 40 holds
-    if (wv != 0 || r >= 8 || r >= M || g >= 2) return;
-#pragma unroll
-    for (int h = 0; h < 2; h++) {
-        uint16_t out[4];
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-            float s = 0.0f, t = 0.0f;
-#pragma unroll
-            for (int k = 0; k < KSPLIT; k++) {
-                s += part[k][h][i][lane] + part[k][h][i][lane + 40];
-                if constexpr (GATED) t += part[k][2 + h][i][lane] + part[k][2 + h][i][lane + 40];
-            }
-            if constexpr (GATED) {
-                const float gv = rnd_l<T>(s), uv = rnd_l<T>(t);
-                const float a = rnd_l<T>(gv / (1.0f + __expf(-gv)));
-                out[i] = f2lo<T>(a * uv);
-            } else {
-                if (bias) s += lo2f<T>(bias[n0 + 8 * h + 4 * g + i]);
-                out[i] = f2lo<T>(s);
-            }
-        }
-        *reinterpret_cast<uint2*>(y + static_cast<size_t>(r) * y_stride + n0 + 8 * h + 4 * g) =
-            make_uint2(static_cast<uint32_t>(out[0]) | (static_cast<uint32_t>(out[1]) << 16),
-                       static_cast<uint32_t>(out[2]) | (static_cast<uint32_t>(out[3]) << 16));
-    }
-}
 
 // The fused q|k|v projection of a decode step with RoPE and the cache appends in its epilogue (M <= 8):
 // small_m8_linear_kernel's loop on the concatenated [(N + 2 Nk) * 128, K] weight, with the workgroup's two
@@ -431,7 +182,7 @@ int launch_small_m_linear(const void* x, int64_t x_stride, const void* w, const 
     dim3 grid(N / 16), block(kWave * ks);
 #define PQ_LAUNCH_L(KERNEL, T, KS, G, S)                                                                             \
     hipLaunchKernelGGL((KERNEL<T, KS, G, S>), grid, block, 0, st, (const uint16_t*)x, x_stride,                      \
-                       (const uint16_t*)w, (const uint16_t*)w_up, (const uint16_t*)bias, (uint16_t*)y, y_stride, M, K)
+                       (const uint16_t*)w, (const uint16_t*)w_up, (const uint16_t*)bias, (uint16_t*)y, y_stride, M, K, HeadEpi{})
 #define PQ_LAUNCH_M8(T, G)                                                                                           \
     do {                                                                                                             \
         if (ks == 8) PQ_LAUNCH_L(small_m8_linear_kernel, T, 8, G, 2);                                                \
