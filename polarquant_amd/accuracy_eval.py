@@ -1,4 +1,4 @@
-"""LongBench and GSM8K runs with the polar-key models, as the reference's scripts make them
+"""LongBench and GSM8K runs with the package's models, as the reference's scripts make them
 (test4long.py, test4gsm8k.py): build the prompt, cut over-long prompts in the middle, generate
 greedily with the reference's decoding loop, score with the reference's metrics, write one JSON
 line per example.  One process, one GPU (the reference spreads the examples over processes with
@@ -26,6 +26,7 @@ import torch
 
 from . import eval_metrics as metrics
 from .modeling_common import generate
+from .registry import family_of
 
 LONGBENCH_DATASETS = ("narrativeqa", "qasper", "multifieldqa_en", "2wikimqa", "hotpotqa", "musique", "lcc", "repobench-p")
 CODE_DATASETS = ("lcc", "repobench-p")          # completed as plain text, without a chat template (test4long.py:110)
@@ -179,7 +180,11 @@ def _load(args) -> Tuple:
     from transformers import AutoTokenizer
     from .checkpoint import load_generation_config, load_pretrained
     tokenizer = AutoTokenizer.from_pretrained(args.model, use_fast=True)
-    options = dict(rbits=args.rbits, tbits=args.tbits, vbits=4 if args.variant == "mixed" else 16, snapkv=args.variant == "snapkv")
+    with open(os.path.join(args.model, "config.json")) as f:
+        family = family_of(json.load(f))
+    options = {}
+    if family.polar_cache:
+        options = dict(rbits=args.rbits, tbits=args.tbits, vbits=4 if args.variant == "mixed" else 16, snapkv=args.variant == "snapkv")
     model = load_pretrained(args.model, torch.bfloat16, "cuda:0", **options)
     return model, tokenizer, load_generation_config(args.model)
 
@@ -193,7 +198,7 @@ def main(argv=None):
         p.add_argument("--data", required=True)
         p.add_argument("--out", required=True)
         p.add_argument("--variant", choices=("polar", "mixed", "snapkv"), default="polar",
-                       help="polar keys; polar keys + 4-bit values; SnapKV prompt eviction in front of polar keys")
+                       help="of the models with a polar-key cache: polar keys; polar keys + 4-bit values; SnapKV prompt eviction in front of polar keys")
         p.add_argument("--rbits", type=int, default=4)
         p.add_argument("--tbits", type=int, default=4)
         p.add_argument("--limit", type=int, default=None, help="only the first N examples of each file")

@@ -111,6 +111,17 @@ def build_latent(verbose: bool = True) -> str:
     return LATENT_LIB
 
 
+LIBRARIES = {"hip": LIB, "latent": LATENT_LIB}
+
+
+def ensure(libraries, verbose: bool = True) -> None:
+    """Build those of the named LIBRARIES that are not there, and nothing else."""
+    if "hip" in libraries and not os.path.exists(LIB):
+        build(verbose)
+    if "latent" in libraries and not os.path.exists(LATENT_LIB):
+        build_latent(verbose)
+
+
 def build(verbose: bool = True, phase_timers: bool = False) -> str:
     """The library the package loads; or, with phase_timers, a second library (same ABI, not loaded by default)
     whose attention kernel times its phases with the wall clock and prints them: a measuring build for

@@ -20,6 +20,7 @@ from typing import Dict, Iterable, List, Optional
 import torch
 
 from .modeling_common import GenerationConfig, PolarConfig
+from .registry import family_of
 
 _ARCH_FIELDS = ("hidden_size", "num_attention_heads", "num_key_value_heads", "num_hidden_layers", "intermediate_size",
                 "vocab_size", "rms_norm_eps", "rope_theta", "rope_scaling", "head_dim", "attention_bias", "mlp_bias",
@@ -33,7 +34,7 @@ def _as_id_list(ids) -> List[int]:
 
 
 def config_from_hf(hf: Dict, **polar_options) -> PolarConfig:
-    """PolarConfig from the dict of a checkpoint's config.json.  `polar_options`: the cache fields of PolarConfig
+    """PolarConfig from the dict of a Llama, Mistral or Qwen2 checkpoint's config.json.  `polar_options`: the cache fields of PolarConfig
     (rbits, tbits, vbits, snapkv, packed_codes, eager_gpu_codes, cache_capacity)."""
     kind = hf.get("model_type", "llama")
     if kind not in ("llama", "qwen2", "mistral"):
@@ -77,12 +78,18 @@ def _shard_files(path: str) -> List[str]:
     raise FileNotFoundError("polarquant_amd: no model.safetensors(.index.json) in %s (pickle checkpoints are not read)" % path)
 
 
+def _named_tensors(model: torch.nn.Module) -> Dict[str, torch.nn.Parameter]:
+    """Checkpoint tensor name -> parameter: the module paths, unless the model maps its names itself."""
+    own = getattr(model, "checkpoint_tensors", None)
+    return own() if own is not None else dict(model.named_parameters())
+
+
 def load_state(model: torch.nn.Module, shard_files: Iterable[str], dtype: torch.dtype) -> None:
     """Copy the tensors of the shards into `model`'s parameters (cast to `dtype`), shard by shard so that host
     memory holds one shard at a time; every parameter must be found, and every tensor must belong to a parameter
     (rotary `inv_freq` buffers that old checkpoints carry are ignored: they are recomputed)."""
     from safetensors import safe_open
-    params = dict(model.named_parameters())
+    params = _named_tensors(model)
     tied = getattr(model.config, "tie_word_embeddings", False)
     seen = set()
     with torch.no_grad():
@@ -107,22 +114,19 @@ def load_state(model: torch.nn.Module, shard_files: Iterable[str], dtype: torch.
         raise KeyError("polarquant_amd: the checkpoint has no tensor for %s" % missing[:8])
 
 
-def load_pretrained(path: str, dtype: torch.dtype = torch.bfloat16, device="cuda:0", model_class=None, **polar_options):
-    """-> the polar-key model of the checkpoint in `path`, in eval mode on `device`.  `model_class`: by default
-    LlamaPolarForCausalLM (also for Mistral, whose layers are Llama's) or Qwen2PolarForCausalLM by `model_type`."""
+def load_pretrained(path: str, dtype: torch.dtype = torch.bfloat16, device="cuda:0", model_class=None, **options):
+    """-> the model of the checkpoint in `path`, in eval mode on `device`, of the family its config.json names (see
+    registry.py) unless `model_class` is given.  `options`: cache options of the family's configuration (the polar-key
+    cache's fields of PolarConfig; `cache_capacity` for every family)."""
     with open(os.path.join(path, "config.json")) as f:
-        hf = json.load(f)
-    cfg = config_from_hf(hf, **polar_options)
-    if model_class is None:
-        if hf.get("model_type") == "qwen2":
-            from .modeling_qwen_polar import Qwen2PolarForCausalLM as model_class
-        else:
-            from .modeling_llama_polar import LlamaPolarForCausalLM as model_class
+        d = json.load(f)
+    family = family_of(d)
+    cfg = family.config(d, **options)
     prev = torch.get_default_dtype()
     torch.set_default_dtype(dtype)
     try:
         with torch.device(device):
-            model = model_class(cfg)
+            model = (model_class or family.model_class())(cfg)
     finally:
         torch.set_default_dtype(prev)
     load_state(model, _shard_files(path), dtype)
@@ -153,15 +157,18 @@ def save_pretrained(model: torch.nn.Module, path: str, model_type: str = "llama"
     from safetensors.torch import save_file
     os.makedirs(path, exist_ok=True)
     c = model.config
-    hf = {k: getattr(c, k) for k in _ARCH_FIELDS if getattr(c, k, None) is not None}
-    hf.update(model_type=model_type, eos_token_id=_as_id_list(getattr(c, "eos_token_id", None)))
+    if hasattr(c, "to_dict"):                       # a configuration that writes its own config.json
+        hf = c.to_dict()
+    else:
+        hf = {k: getattr(c, k) for k in _ARCH_FIELDS if getattr(c, k, None) is not None}
+        hf.update(model_type=model_type, eos_token_id=_as_id_list(getattr(c, "eos_token_id", None)))
     with open(os.path.join(path, "config.json"), "w") as f:
         json.dump(hf, f, indent=1)
-    g = generation or GenerationConfig(eos_token_id=hf["eos_token_id"] or [2])
+    g = generation or GenerationConfig(eos_token_id=hf.get("eos_token_id") or [2])
     with open(os.path.join(path, "generation_config.json"), "w") as f:
         json.dump(dataclasses.asdict(g), f, indent=1)
     tied = getattr(c, "tie_word_embeddings", False)
-    state = {k: v.detach().cpu().contiguous() for k, v in model.named_parameters() if not (tied and k == "lm_head.weight")}
+    state = {k: v.detach().cpu().contiguous() for k, v in _named_tensors(model).items() if not (tied and k == "lm_head.weight")}
     names = list(state)
     if shards <= 1:
         save_file(state, os.path.join(path, "model.safetensors"))

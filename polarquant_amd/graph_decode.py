@@ -27,7 +27,46 @@ from .attention import _num_cus, new_workspace, plan_splits, polar_decode_attent
 from .modeling_common import GROUP, apply_rotary_pos_emb
 
 
-class PolarGraphDecoder:
+class GraphDecoder:
+    """Capture and replay of a one-token step whose every input and output is static device state."""
+
+    model = None
+    use_graph = True
+    graph: Optional[torch.cuda.CUDAGraph] = None
+    logits: Optional[torch.Tensor] = None
+
+    def _step_body(self) -> torch.Tensor:
+        raise NotImplementedError
+
+    def _step_state(self) -> List[torch.Tensor]:
+        """The tensors a step changes in a way that running it again would not reproduce."""
+        raise NotImplementedError
+
+    def _run_step(self) -> torch.Tensor:
+        if not self.use_graph:
+            return self._step_body()
+        if self.graph is None:
+            # warm up on a side stream (lazy library initialisation must not be captured), then capture;
+            # the warm-up step advances the state, so it is put back before and after
+            state = self._step_state()
+            saved = [t.clone() for t in state]
+            s = torch.cuda.Stream()
+            s.wait_stream(torch.cuda.current_stream())
+            with torch.cuda.stream(s):
+                self._step_body()
+            torch.cuda.current_stream().wait_stream(s)
+            for t, v in zip(state, saved):
+                t.copy_(v)
+            self.graph = torch.cuda.CUDAGraph()
+            with torch.cuda.graph(self.graph):
+                self.logits = self._step_body()
+            for t, v in zip(state, saved):
+                t.copy_(v)
+        self.graph.replay()
+        return self.logits
+
+
+class PolarGraphDecoder(GraphDecoder):
     def __init__(self, model, max_len: int, use_graph: bool = True, fused_ops: bool = True, small_m_gemm: bool = True,
                  fused_prefill: bool = False, fused_qkv_rope: bool = True):
         """fused_ops: run RoPE + cache append, the norms and the MLP activation as one HIP launch each
@@ -268,31 +307,14 @@ class PolarGraphDecoder:
         self.n_groups_dev.add_(1)
         self.n_resid_dev.fill_(1)
 
+    def _step_state(self):
+        return [self.pos, self.resid_idx, self.n_resid_dev]
+
     @torch.no_grad()
     def step(self, ids: torch.Tensor) -> torch.Tensor:
         assert self.kv_len + 1 <= self.max_len, "cache capacity exhausted"
         self.ids.copy_(ids.view(self.B, 1))
-        if self.use_graph:
-            if self.graph is None:
-                # warm up on a side stream (lazy library initialisation must not be captured), then capture;
-                # the warm-up steps advance the counters, so they are put back before and after
-                state = [t.clone() for t in (self.pos, self.resid_idx, self.n_resid_dev)]
-                s = torch.cuda.Stream()
-                s.wait_stream(torch.cuda.current_stream())
-                with torch.cuda.stream(s):
-                    self._step_body()
-                torch.cuda.current_stream().wait_stream(s)
-                for t, v in zip((self.pos, self.resid_idx, self.n_resid_dev), state):
-                    t.copy_(v)
-                self.graph = torch.cuda.CUDAGraph()
-                with torch.cuda.graph(self.graph):
-                    self.logits = self._step_body()
-                for t, v in zip((self.pos, self.resid_idx, self.n_resid_dev), state):
-                    t.copy_(v)
-            self.graph.replay()
-            logits = self.logits
-        else:
-            logits = self._step_body()
+        logits = self._run_step()
         self.kv_len += 1
         self.n_resid += 1
         for ar in self.arenas:
@@ -304,3 +326,48 @@ class PolarGraphDecoder:
     def cache(self):
         """The reference-format cache tuples of the current state (one per layer)."""
         return tuple(ar.as_tuple() for ar in self.arenas)
+
+
+class LatentGraphDecoder(GraphDecoder):
+    """The same for latent-attention models (`modeling_latent`): the step is the model's own `run` for one token, with the
+    position in device memory."""
+
+    def __init__(self, model, max_len: int, use_graph: bool = True):
+        self.model, self.max_len, self.use_graph = model, int(max_len), use_graph
+
+    @torch.no_grad()
+    def prefill(self, input_ids: torch.Tensor, attention_mask: Optional[torch.Tensor] = None) -> torch.Tensor:
+        from .latent_ops import decode_splits
+        B, L = input_ids.shape
+        assert L + 1 <= self.max_len
+        out = self.model(input_ids=input_ids, attention_mask=attention_mask, num_logits_to_keep=1,
+                         past_key_values=self.model.new_cache(B, self.max_len))      # never grows: the graph keeps its addresses
+        self.arenas = [t.arena for t in out.past_key_values]
+        self.B, self.kv_len, self.graph, self.logits = B, L, None, None
+        dev = input_ids.device
+        self.pos = torch.full((1,), L, dtype=torch.int32, device=dev)
+        self.ids = torch.zeros((B, 1), dtype=torch.long, device=dev)
+        self.n_splits = [decode_splits(B, 1, layer.mix.heads, self.max_len, dev) for layer in self.model.model.layers]
+        return out.logits
+
+    def _step_state(self):
+        return [self.pos] + [s.rows for a in self.arenas for s in a.conv]
+
+    def _step_body(self):
+        h = self.model.model.run(self.ids, self.arenas, 0, self.pos, self.n_splits)
+        logits = self.model.logits(h)
+        self.pos.add_(1)
+        return logits
+
+    @torch.no_grad()
+    def step(self, ids: torch.Tensor) -> torch.Tensor:
+        assert self.kv_len + 1 <= self.max_len, "cache capacity exhausted"
+        self.ids.copy_(ids.view(self.B, 1))
+        logits = self._run_step()
+        self.kv_len += 1
+        for a in self.arenas:
+            a.kv_len = self.kv_len
+        return logits
+
+    def cache(self):
+        return tuple(a.as_tuple() for a in self.arenas)

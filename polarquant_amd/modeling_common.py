@@ -709,6 +709,11 @@ class PolarForCausalLM(nn.Module):
     def _prepare_cache_for_generation(self, *args, **kwargs):
         return None                      # the cache is this model's own tuple, never an HF cache object (:562-563)
 
+    def graph_decoder(self, max_len: int):
+        """The decoder that replays this model's one-token step from a captured HIP graph."""
+        from .graph_decode import PolarGraphDecoder
+        return PolarGraphDecoder(self, max_len=max_len)
+
     def kv_cache_bytes_per_token(self) -> int:
         """Bytes one cached token costs across all layers: 1 code byte per pair, 4 metadata
         halves per (group, pair) amortised over 128 tokens, fp16 V (or 4-bit V with config.vbits == 4)."""
@@ -773,7 +778,7 @@ def generate(model, input_ids, attention_mask, generation_config, do_sample=Fals
     the mask grown by a column of ones; stops early once every sequence has produced a stop token (sequences that
     stopped earlier keep producing tokens until then, as in the reference).  -> LongTensor [B, <= max_new_tokens].
     graph_decoder (not in the reference): the steps after the prompt replay a captured HIP graph on static state
-    (`graph_decode.PolarGraphDecoder`) instead of driving the modules launch by launch; logits agree with the
+    (the model's `graph_decoder`) instead of driving the modules launch by launch; logits agree with the
     eager step to rounding, so a near-tie between two tokens may resolve differently."""
     dev = model.device
     n_seq = input_ids.size(0)
@@ -784,8 +789,7 @@ def generate(model, input_ids, attention_mask, generation_config, do_sample=Fals
     tokens, cache, n_out = input_ids, None, 0
     decoder = None
     if graph_decoder:
-        from .graph_decode import PolarGraphDecoder
-        decoder = PolarGraphDecoder(model, max_len=input_ids.size(1) + max_new_tokens + 1)
+        decoder = model.graph_decoder(max_len=input_ids.size(1) + max_new_tokens + 1)
     with torch.no_grad():
         while n_out < max_new_tokens:
             if decoder is None:
