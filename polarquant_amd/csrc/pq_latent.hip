@@ -300,7 +300,7 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(LatentNormArgs a) {
 }
 
 int launch_latent_norm(const LatentNormArgs& a, int dtype, hipStream_t st) {
-    const bool v4 = a.q_rank % 4 == 0 && a.kv_rank % 4 == 0 && a.row_stride % 4 == 0;
+    const bool v4 = a.q_rank % 4 == 0 && (!a.w_kv || a.kv_rank % 4 == 0) && a.row_stride % 4 == 0;
     dim3 grid(static_cast<unsigned>(a.B * a.L)), block(256);
 #define PQ_LN(T) do { if (v4) hipLaunchKernelGGL((latent_norm_kernel<T, 4>), grid, block, 0, st, a); \
                       else hipLaunchKernelGGL((latent_norm_kernel<T, 1>), grid, block, 0, st, a); } while (0)
