@@ -363,6 +363,9 @@ def main():
     ap.add_argument("--no-values4", action="store_true", help="skip the 4-bit-value (Mixed variant) measurement")
     ap.add_argument("--no-configs", action="store_true", help="skip configs[0], [2], [3] and [4]")
     ap.add_argument("--no-ramp", action="store_true", help="no clock ramp before the timed regions (counter-collection runs under the profiler)")
+    ap.add_argument("--dekipel", action="store_true",
+                    help="instead of the headline workload: prompt and decode throughput of the Dekipel decoder, and its kernels, beside the "
+                         "Llama shell with the polar-key cache at equal size (one JSON line per figure)")
     ap.add_argument("--copy-calib", action="store_true",
                     help="also run 3 plain 1 GiB device copies (torch clone): under `rocprofv3 --pmc FETCH_SIZE|WRITE_SIZE` "
                          "their counter values give the scale factor for the attention kernel's")
@@ -375,6 +378,10 @@ def main():
         print("bench.py: no GPU visible", file=sys.stderr)
         sys.exit(1)
 
+    if args.dekipel:
+        from polarquant_amd.benchmarks import latent_bench
+        latent_bench.main([])
+        return
     from polarquant_amd import _ffi, workloads as wl
     if args.no_ramp:
         wl.RAMP_SECONDS = 0.0

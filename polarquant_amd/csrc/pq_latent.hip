@@ -50,10 +50,13 @@ template <typename T, int V> __device__ __forceinline__ void stv(void* base, siz
     }
 }
 
+// sum over the wavefront, in every lane: rotations inside rows of 16 lanes, then the four rows' sums through scalars
 __device__ __forceinline__ float wave_sum(float v) {
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
-    return v;
+    v += __uint_as_float(row_rotate<8>(__float_as_uint(v)));
+    v += __uint_as_float(row_rotate<4>(__float_as_uint(v)));
+    v += __uint_as_float(row_rotate<2>(__float_as_uint(v)));
+    v += __uint_as_float(row_rotate<1>(__float_as_uint(v)));
+    return (readlane_f(v, 0) + readlane_f(v, 16)) + (readlane_f(v, 32) + readlane_f(v, 48));
 }
 
 // ---- residual add + grouped norms + causal convolution ----------------------------------------------------------------
@@ -66,26 +69,46 @@ __device__ __forceinline__ float wave_sum(float v) {
 // Sums over a group: where every wavefront's piece lies in one group (`wave_groups`), wavefront sums go through LDS once;
 // otherwise every piece's sum does, and wavefronts add them up group by group.
 template <typename T, int TAPS, int V, int NC>
-__global__ __launch_bounds__(1024) void norm_conv_kernel(NormConvArgs a) {
-    extern __shared__ float lds[];
+__global__ __launch_bounds__(512) void norm_conv_kernel(NormConvArgs a) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
     const int tid = threadIdx.x, nthr = blockDim.x, nw = nthr / kWave, wv = tid / kWave, lane = tid & (kWave - 1);
     const int b = blockIdx.y, W = a.W, L = a.L, taps = a.taps;
     const int t0 = blockIdx.x * a.strip, t1 = t0 + a.strip < L ? t0 + a.strip : L;
     const int gs = W / a.groups, pieces = W / V, ppg = gs / V;       // pieces, pieces per group
-    const bool wave_groups = a.groups == 1 || (ppg % kWave) == 0;
-    const int spg = a.groups == 1 ? NC * nw : ppg / kWave;           // wavefront slots per group
+    const bool one_group = a.groups == 1, wave_groups = one_group || (ppg % kWave) == 0;
+    const int spg = one_group ? nw : ppg / kWave;                    // wavefront sums per group
     const float inv_gs = 1.0f / static_cast<float>(gs);
-    const size_t row0 = static_cast<size_t>(b) * L;
+    const int begin = (TAPS > 0 && t0 > 0) ? t0 - (taps - 1) : t0;   // strips are longer than the filter
     int phase = 0;
 
     bool own[NC];
-    int ch[NC];
+    uint32_t ch[NC];
 #pragma unroll
     for (int k = 0; k < NC; k++) {
         const int q = k * nthr + tid;
         own[k] = q < pieces;
         ch[k] = (own[k] ? q : 0) * V;
     }
+    // rows of this sequence; without y something that exists is loaded in its place and not used
+    const float* xr = a.x_in + static_cast<size_t>(b) * L * W;
+    const elem_t<T>* yr = a.y ? static_cast<const elem_t<T>*>(a.y) + static_cast<size_t>(b) * L * W : static_cast<const elem_t<T>*>(a.w_pre);
+    const size_t y_stride = a.y ? W : 0;
+    // tokens in flight ahead of the one being worked on: what a compute unit holds of them is what keeps HBM busy
+    constexpr int AHEAD = NC == 1 ? 3 : 1;
+    float xc[NC][V], yc[NC][V], xn[AHEAD][NC][V], yn[AHEAD][NC][V];
+    auto fetch = [&](int t, float (&x)[NC][V], float (&y)[NC][V]) {
+        const float* xp = xr + static_cast<size_t>(t) * W;
+        const elem_t<T>* yp = yr + t * y_stride;
+#pragma unroll
+        for (int k = 0; k < NC; k++) {
+            ldv<F32, V>(xp, ch[k], x[k]);
+            ldv<T, V>(yp, ch[k], y[k]);
+        }
+    };
+    fetch(begin, xc, yc);
+#pragma unroll
+    for (int d = 0; d < AHEAD; d++) fetch(begin + d + 1 < t1 ? begin + d + 1 : begin, xn[d], yn[d]);
+
     // 1 / sqrt(mean square of the group + eps) for each of this thread's pieces
     auto group_scale = [&](const float (&v)[NC][V], float (&r)[NC]) {
         float s[NC];
@@ -97,19 +120,34 @@ __global__ __launch_bounds__(1024) void norm_conv_kernel(NormConvArgs a) {
             if (!own[k]) s[k] = 0.0f;
         }
         if (wave_groups) {
-            float* buf = lds + (phase & 1) * (NC * nw);
+            float* buf = lds + (phase & 1) * (NC * 8);
             phase++;
+            if (one_group) {
 #pragma unroll
-            for (int k = 0; k < NC; k++) {
-                const float ws = wave_sum(s[k]);
-                if (lane == 0) buf[k * nw + wv] = ws;
+                for (int k = 1; k < NC; k++) s[0] += s[k];
+                s[0] = wave_sum(s[0]);
+                if (lane == 0) buf[wv] = s[0];
+            } else {
+#pragma unroll
+                for (int k = 0; k < NC; k++) {
+                    const float ws = wave_sum(s[k]);
+                    if (lane == 0) buf[k * nw + wv] = ws;
+                }
             }
             __syncthreads();
 #pragma unroll
             for (int k = 0; k < NC; k++) {
-                const int slot = k * nw + wv, first = (slot / spg) * spg;
+                if (k > 0 && one_group) { r[k] = r[0]; continue; }
+                const int slot = k * nw + wv, slots = one_group ? nw : NC * nw, group = one_group ? 0 : slot / spg;
                 float sum = 0.0f;
-                for (int j = 0; j < spg; j++) sum += buf[first + j < NC * nw ? first + j : 0];
+                if ((spg & 3) == 0 && (group + 1) * spg <= slots) {
+                    for (int j = 0; j < spg; j += 4) {
+                        const float4 p = *reinterpret_cast<const float4*>(buf + group * spg + j);
+                        sum += (p.x + p.y) + (p.z + p.w);
+                    }
+                } else {
+                    for (int j = 0; j < spg; j++) sum += buf[group * spg + j < slots ? group * spg + j : 0];
+                }
                 r[k] = rsqrtf(sum * inv_gs + a.eps);
             }
         } else {
@@ -136,56 +174,65 @@ __global__ __launch_bounds__(1024) void norm_conv_kernel(NormConvArgs a) {
 #pragma unroll
     for (int k = 0; k < NC; k++) {
         ldv<T, V>(a.w_pre, ch[k], wpre[k]);
-        if (a.y) ldv<T, V>(a.w_post, ch[k], wpost[k]);
+        ldv<T, V>(a.y ? a.w_post : a.w_pre, ch[k], wpost[k]);
     }
+    // (loads of what a shorter filter or a later strip does not have go to an address that exists and are dropped: with a
+    // branch around each, every one would be waited for before the next)
     if constexpr (TAPS > 0) {
         const elem_t<T>* w = static_cast<const elem_t<T>*>(a.conv_w);
-#pragma unroll
-        for (int j = 0; j < TAPS; j++) {
-            const int tap = j - (TAPS - taps);               // of the real filter; negative: padding
+        if (taps == TAPS && V == 4 && TAPS % 4 == 0) {
 #pragma unroll
             for (int k = 0; k < NC; k++)
 #pragma unroll
-                for (int i = 0; i < V; i++) cw[j][k][i] = tap >= 0 ? ld1<T>(w + static_cast<size_t>(ch[k] + i) * taps + tap) : 0.0f;
+                for (int i = 0; i < V; i++)
+#pragma unroll
+                    for (int j = 0; j + 4 <= TAPS; j += 4) {
+                        float c4[4];
+                        ldv<T, 4>(w, (ch[k] + i) * static_cast<size_t>(TAPS) + j, c4);
+#pragma unroll
+                        for (int jj = 0; jj < 4; jj++) cw[j + jj][k][i] = c4[jj];
+                    }
+        } else {
+#pragma unroll
+            for (int j = 0; j < TAPS; j++) {
+                const int tap = j - (TAPS - taps);           // of the real filter; negative: padding
+#pragma unroll
+                for (int k = 0; k < NC; k++)
+#pragma unroll
+                    for (int i = 0; i < V; i++) {
+                        const float c1 = ld1<T>(w + (ch[k] + i) * static_cast<size_t>(taps) + (tap >= 0 ? tap : 0));
+                        cw[j][k][i] = tap >= 0 ? c1 : 0.0f;
+                    }
+            }
         }
+        const float* state = taps > 1 ? a.state_in : a.x_in;
 #pragma unroll
         for (int j = 0; j < TAPS - 1; j++) {
             const int row = j - (TAPS - taps);
 #pragma unroll
             for (int k = 0; k < NC; k++) {
-                if (t0 == 0 && row >= 0)
-                    ldv<F32, V>(a.state_in, (static_cast<size_t>(b) * (taps - 1) + row) * W + ch[k], ring[j][k]);
-                else
+                ldv<F32, V>(state, (static_cast<size_t>(b) * (taps - 1) + (row >= 0 ? row : 0)) * W + ch[k], ring[j][k]);
+                const bool has = t0 == 0 && row >= 0;
 #pragma unroll
-                    for (int i = 0; i < V; i++) ring[j][k][i] = 0.0f;
+                for (int i = 0; i < V; i++) ring[j][k][i] = has ? ring[j][k][i] : 0.0f;
             }
         }
     }
     const int first_tok = a.start ? a.start[b] - (a.pos_dev ? *a.pos_dev : a.pos) : 0;      // tokens before it are padding
-    const int begin = (TAPS > 0 && t0 > 0) ? t0 - (taps - 1) : t0;      // strips are longer than the filter
 
-    float xc[NC][V], yc[NC][V], xn[NC][V], yn[NC][V];
-    auto fetch = [&](int t, float (&x)[NC][V], float (&y)[NC][V]) {
-#pragma unroll
-        for (int k = 0; k < NC; k++) {
-            ldv<F32, V>(a.x_in, (row0 + t) * W + ch[k], x[k]);
-            if (a.y) ldv<T, V>(a.y, (row0 + t) * W + ch[k], y[k]);
-        }
-    };
-    fetch(begin, xc, yc);
     for (int t = begin; t < t1; t++) {
-        if (t + 1 < t1) fetch(t + 1, xn, yn);
+        const size_t row = (static_cast<size_t>(b) * L + t) * W;
         if (a.y) {
             float r[NC];
             group_scale(yc, r);
 #pragma unroll
             for (int k = 0; k < NC; k++)
 #pragma unroll
-                for (int i = 0; i < V; i++) xc[k][i] += wpost[k][i] * (yc[k][i] * r[k]);
-            if (t >= t0 && a.x_out)
+                for (int i = 0; i < V; i++) xc[k][i] = __builtin_fmaf(wpost[k][i], yc[k][i] * r[k], xc[k][i]);
+            if (t >= t0)
 #pragma unroll
                 for (int k = 0; k < NC; k++)
-                    if (own[k]) stv<F32, V>(a.x_out, (row0 + t) * W + ch[k], xc[k]);
+                    if (own[k]) stv<F32, V>(a.x_out + row, ch[k], xc[k]);
         }
         float r[NC];
         group_scale(xc, r);
@@ -204,18 +251,24 @@ __global__ __launch_bounds__(1024) void norm_conv_kernel(NormConvArgs a) {
                     float c = cw[TAPS - 1][k][i] * h[i];
 #pragma unroll
                     for (int j = 0; j < TAPS - 1; j++) c = __builtin_fmaf(cw[j][k][i], ring[j][k][i], c);
-                    if (real) o[i] += c;
+                    o[i] += real ? c : 0.0f;
 #pragma unroll
                     for (int j = 0; j + 1 < TAPS - 1; j++) ring[j][k][i] = ring[j + 1][k][i];
                     if constexpr (TAPS > 1) ring[TAPS > 1 ? TAPS - 2 : 0][k][i] = h[i];
                 }
             }
-            if (t >= t0 && own[k]) stv<T, V>(a.h_out, (row0 + t) * W + ch[k], o);
+            if (t >= t0 && own[k]) stv<T, V>(static_cast<elem_t<T>*>(a.h_out) + row, ch[k], o);
         }
 #pragma unroll
         for (int k = 0; k < NC; k++)
 #pragma unroll
-            for (int i = 0; i < V; i++) { xc[k][i] = xn[k][i]; yc[k][i] = yn[k][i]; }
+            for (int i = 0; i < V; i++) {
+                xc[k][i] = xn[0][k][i];
+                yc[k][i] = yn[0][k][i];
+#pragma unroll
+                for (int d = 0; d + 1 < AHEAD; d++) { xn[d][k][i] = xn[d + 1][k][i]; yn[d][k][i] = yn[d + 1][k][i]; }
+            }
+        fetch(t + AHEAD + 1 < t1 ? t + AHEAD + 1 : t, xn[AHEAD - 1], yn[AHEAD - 1]);
     }
     if constexpr (TAPS > 1) {
         if (t1 == L) {
@@ -225,7 +278,7 @@ __global__ __launch_bounds__(1024) void norm_conv_kernel(NormConvArgs a) {
                 if (row < 0) continue;
 #pragma unroll
                 for (int k = 0; k < NC; k++)
-                    if (own[k]) stv<F32, V>(a.state_out, (static_cast<size_t>(b) * (taps - 1) + row) * W + ch[k], ring[j][k]);
+                    if (own[k]) stv<F32, V>(a.state_out + (static_cast<size_t>(b) * (taps - 1) + row) * W, ch[k], ring[j][k]);
             }
         }
     }
@@ -237,16 +290,20 @@ int launch_norm_conv(const NormConvArgs& args, int dtype, hipStream_t st) {
     if (!a.conv_w) a.taps = 1;
     const int V = ((a.W / a.groups) % 4 == 0) ? 4 : 1;
     const int pieces = a.W / V;
-    const int nthr = pieces <= 256 ? 256 : pieces <= 512 ? 512 : 1024;
+    const int nthr = pieces <= 256 ? 256 : 512;
     const int per = (pieces + nthr - 1) / nthr;
-    const int NC = per <= 1 ? 1 : per <= 2 ? 2 : 4;
-    if (per > 4) return static_cast<int>(hipErrorInvalidValue);
+    const int NC = per <= 1 ? 1 : per <= 2 ? 2 : per <= 4 ? 4 : 8;
+    if (per > 8) return static_cast<int>(hipErrorInvalidValue);
     a.strip = a.L <= kConvInPlaceTokens ? a.L : 32;
-    const size_t shared = (static_cast<size_t>(NC) * nthr + a.groups + 2 * NC * (nthr / kWave)) * sizeof(float);
+    const size_t shared = (static_cast<size_t>(NC) * nthr + a.groups) * sizeof(float);
     if (shared > 64 * 1024) return static_cast<int>(hipErrorInvalidValue);
     dim3 grid(static_cast<unsigned>((a.L + a.strip - 1) / a.strip), static_cast<unsigned>(a.B)), block(nthr);
 #define PQ_NC(T, TP, VV, N) hipLaunchKernelGGL((norm_conv_kernel<T, TP, VV, N>), grid, block, shared, st, a)
-#define PQ_NC_N(T, TP, VV) do { if (NC == 1) PQ_NC(T, TP, VV, 1); else if (NC == 2) PQ_NC(T, TP, VV, 2); else PQ_NC(T, TP, VV, 4); } while (0)
+#define PQ_NC_N(T, TP, VV)                                                                                           \
+    do {                                                                                                             \
+        if (NC == 1) PQ_NC(T, TP, VV, 1); else if (NC == 2) PQ_NC(T, TP, VV, 2);                                     \
+        else if (NC == 4) PQ_NC(T, TP, VV, 4); else PQ_NC(T, TP, VV, 8);                                             \
+    } while (0)
 #define PQ_NC_V(T, TP) do { if (V == 4) PQ_NC_N(T, TP, 4); else PQ_NC_N(T, TP, 1); } while (0)
 #define PQ_NC_T(T)                                                                                                   \
     do {                                                                                                             \
@@ -264,48 +321,62 @@ int launch_norm_conv(const NormConvArgs& args, int dtype, hipStream_t st) {
 }
 
 // ---- norms of the two latents ---------------------------------------------------------------------------------------
-// One workgroup per token.
-template <typename T, int V>
+// A wavefront per token when there are many (WIDE false), a workgroup per token otherwise.
+template <typename T, int V, bool WIDE>
 __global__ __launch_bounds__(256) void latent_norm_kernel(LatentNormArgs a) {
     __shared__ float part[2][4];
-    const int tok = blockIdx.x, b = tok / a.L, t = tok - b * a.L, tid = threadIdx.x;
+    const int wv = threadIdx.x >> 6, n_tok = a.B * a.L;
+    const int first = (WIDE ? static_cast<int>(threadIdx.x) : static_cast<int>(threadIdx.x & 63)) * V, step = (WIDE ? 256 : 64) * V;
+    int tok = WIDE ? static_cast<int>(blockIdx.x) : static_cast<int>(blockIdx.x) * 4 + wv;
+    if (!WIDE && tok >= n_tok) return;
+    const int b = tok / a.L, t = tok - b * a.L;
     const int Q = a.q_rank, R = a.w_kv ? a.kv_rank : 0;
-    const size_t in = static_cast<size_t>(tok) * a.row_stride;
+    const elem_t<T>* p = static_cast<const elem_t<T>*>(a.p) + static_cast<size_t>(tok) * a.row_stride;
     float sq = 0.0f, sc = 0.0f, v[V];
-    for (int i = tid * V; i < Q + R; i += 256 * V) {
-        ldv<T, V>(a.p, in + i, v);
+    for (int i = first; i < Q + R; i += step) {
+        ldv<T, V>(p, i, v);
         float s = 0.0f;
 #pragma unroll
         for (int j = 0; j < V; j++) s = __builtin_fmaf(v[j], v[j], s);
-        if (i < Q) sq += s; else sc += s;
+        sq += i < Q ? s : 0.0f;
+        sc += i < Q ? 0.0f : s;
     }
     sq = wave_sum(sq);
     sc = wave_sum(sc);
-    if ((tid & 63) == 0) { part[0][tid >> 6] = sq; part[1][tid >> 6] = sc; }
-    __syncthreads();
-    const float rq = rsqrtf((part[0][0] + part[0][1] + part[0][2] + part[0][3]) / static_cast<float>(Q) + a.eps);
-    const float rc = R ? rsqrtf((part[1][0] + part[1][1] + part[1][2] + part[1][3]) / static_cast<float>(R) + a.eps) : 0.0f;
+    if (WIDE) {
+        if ((threadIdx.x & 63) == 0) { part[0][wv] = sq; part[1][wv] = sc; }
+        __syncthreads();
+        sq = part[0][0] + part[0][1] + part[0][2] + part[0][3];
+        sc = part[1][0] + part[1][1] + part[1][2] + part[1][3];
+    }
+    const float rq = rsqrtf(sq / static_cast<float>(Q) + a.eps), rc = R ? rsqrtf(sc / static_cast<float>(R) + a.eps) : 0.0f;
     int64_t pos = (a.pos_dev ? *a.pos_dev : a.pos) + t;
     pos = pos < 0 ? 0 : (pos >= a.capacity ? a.capacity - 1 : pos);          // (never past the cache)
-    const size_t qo = static_cast<size_t>(tok) * Q, co = (static_cast<size_t>(b) * a.capacity + pos) * R;
-    for (int i = tid * V; i < Q + R; i += 256 * V) {
+    elem_t<T>* qo = static_cast<elem_t<T>*>(a.q_out) + static_cast<size_t>(tok) * Q;
+    elem_t<T>* co = static_cast<elem_t<T>*>(a.cache) + (static_cast<size_t>(b) * a.capacity + pos) * R;
+    for (int i = first; i < Q + R; i += step) {
+        const bool is_q = i < Q;
         float w[V];
-        ldv<T, V>(a.p, in + i, v);
-        if (i < Q) ldv<T, V>(a.w_q, i, w); else ldv<T, V>(a.w_kv, i - Q, w);
-        const float r = i < Q ? rq : rc;
+        ldv<T, V>(p, i, v);
+        ldv<T, V>(is_q ? a.w_q : a.w_kv, is_q ? i : i - Q, w);
+        const float r = is_q ? rq : rc;
 #pragma unroll
         for (int j = 0; j < V; j++) v[j] = w[j] * (v[j] * r);
-        if (i < Q) stv<T, V>(a.q_out, qo + i, v); else stv<T, V>(a.cache, co + (i - Q), v);
+        stv<T, V>(is_q ? qo : co, is_q ? i : i - Q, v);
     }
 }
 
 int launch_latent_norm(const LatentNormArgs& a, int dtype, hipStream_t st) {
     const bool v4 = a.q_rank % 4 == 0 && (!a.w_kv || a.kv_rank % 4 == 0) && a.row_stride % 4 == 0;
-    dim3 grid(static_cast<unsigned>(a.B * a.L)), block(256);
-#define PQ_LN(T) do { if (v4) hipLaunchKernelGGL((latent_norm_kernel<T, 4>), grid, block, 0, st, a); \
-                      else hipLaunchKernelGGL((latent_norm_kernel<T, 1>), grid, block, 0, st, a); } while (0)
+    const int n_tok = a.B * a.L;
+    const bool wide = n_tok < 1024;
+    dim3 grid(static_cast<unsigned>(wide ? n_tok : (n_tok + 3) / 4)), block(256);
+#define PQ_LN1(T, V) do { if (wide) hipLaunchKernelGGL((latent_norm_kernel<T, V, true>), grid, block, 0, st, a); \
+                          else hipLaunchKernelGGL((latent_norm_kernel<T, V, false>), grid, block, 0, st, a); } while (0)
+#define PQ_LN(T) do { if (v4) PQ_LN1(T, 4); else PQ_LN1(T, 1); } while (0)
     if (dtype == 0) PQ_LN(F16); else if (dtype == 1) PQ_LN(BF16); else PQ_LN(F32);
 #undef PQ_LN
+#undef PQ_LN1
     return static_cast<int>(hipGetLastError());
 }
 

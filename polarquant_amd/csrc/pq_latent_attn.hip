@@ -51,26 +51,31 @@ template <typename T> __device__ __forceinline__ uint32_t pack2(float a, float b
 }
 
 // ---- decode --------------------------------------------------------------------------------------------------------
-// grid (slices, row tiles, sequences); a row is (query token, head), a wavefront owns 16 of them, RW wavefronts share the
-// latents of a 32-token tile in LDS (double-buffered, next tile's loads in flight over the current tile's products).
-// The same tile serves both products: rows of it (16 bytes per lane) as K, columns of it, transposed on the way out of
-// LDS, as V.  16-byte pieces of a row are XOR-swizzled by the token so that neither access meets in few banks.
+// grid (slices, row tiles, sequences); a row is (query token, head), a workgroup owns 16 * RT of them and walks its slice
+// 32 keys at a time.  The latent's channels are divided among its wavefronts: each holds its channels of the queries and of
+// the output, loads its channels of the keys (the next tile's while it works on the current one) and keeps them in LDS of
+// its own.  Per tile, each wavefront multiplies its channels of K and Q^T, the partial scores are added up through LDS (the
+// only barrier), every wavefront runs the softmax of all rows, and multiplies its channels of V^T, the same LDS tile
+// transposed on the way out, with P^T.  So each key is read from HBM once, and from LDS once per product, for all rows.
+// 16-byte pieces of a key's row are XOR-swizzled by the key so that neither access meets in few banks.
 // Workspace: [B, slices, L * H] pairs (maximum in log2 units, sum), then as many rows of R floats.
 constexpr int kDecodeTile = 32;
 __device__ __forceinline__ size_t pairs_floats(const LatentDecodeArgs& a) {     // up to the accumulators' 16-byte boundary
     return (2 * static_cast<size_t>(a.B) * a.n_splits * a.L * a.H + 3) & ~static_cast<size_t>(3);
 }
+template <int RP> struct DecodeShape {
+    static constexpr int CW = RP / 4 < 32 ? 32 : RP / 4;       // channels per wavefront
+    static constexpr int NW = RP / CW;                         // wavefronts
+};
 
-template <typename T, int RP, int RW>
-__global__ __launch_bounds__(kWave * RW) void latent_decode_kernel(LatentDecodeArgs a) {
-    constexpr int CH = RP / 8, NT = kWave * RW, LPT = kDecodeTile * CH / NT, KS = RP / 32, CT = RP / 16;
-    static_assert(LPT >= 1 && LPT * NT == kDecodeTile * CH, "whole loads");
-    __shared__ __attribute__((aligned(16))) uint16_t tile[2][kDecodeTile * RP];
+template <typename T, int RP, int RT>
+__global__ __launch_bounds__(kWave * DecodeShape<RP>::NW, RT <= 2 ? 2 : 1) void latent_decode_kernel(LatentDecodeArgs a) {
+    constexpr int CW = DecodeShape<RP>::CW, NW = DecodeShape<RP>::NW, CH = CW / 8, KS = CW / 32, CT = CW / 16;
+    constexpr int LPT = kDecodeTile * CH / kWave, RPW = 16 / CH;           // loads per lane; rows per 256 bytes of LDS
+    __shared__ __attribute__((aligned(16))) uint16_t tiles[NW][kDecodeTile * CW];
+    __shared__ floatx4_a exch[2][NW][2 * RT][kWave];
     const int tid = threadIdx.x, lane = tid & 63, wv = tid / kWave, r16 = lane & 15, g = lane >> 4;
-    const int b = blockIdx.z, split = blockIdx.x, R = a.R, rows = a.L * a.H;
-    const int n = blockIdx.y * 16 * RW + wv * 16 + r16;
-    const bool valid = n < rows;
-    const int nc = valid ? n : rows - 1;
+    const int b = blockIdx.z, split = blockIdx.x, R = a.R, rows = a.L * a.H, n0 = blockIdx.y * 16 * RT;
     const int pos = a.pos_dev ? *a.pos_dev : a.pos;
     int64_t total = static_cast<int64_t>(pos) + a.L;
     if (total > a.capacity) total = a.capacity;
@@ -83,138 +88,182 @@ __global__ __launch_bounds__(kWave * RW) void latent_decode_kernel(LatentDecodeA
     float* ml = a.workspace + 2 * part;
     float* acc = a.workspace + pairs_floats(a) + part * R;
     if (s0 >= s1) {                                  // uniform over the workgroup
-        if (valid && g == 0) { ml[2 * n] = kNone; ml[2 * n + 1] = 0.0f; }
+        if (tid < 16 * RT && n0 + tid < rows) { ml[2 * (n0 + tid)] = kNone; ml[2 * (n0 + tid) + 1] = 0.0f; }
         return;
     }
-    auto swz = [](int tok) { return RP >= 128 ? (tok & 15) : ((tok >> 1) & 7); };
+    auto swz = [](int tok) { return (tok / RPW) % CH; };
+    const int c0 = wv * CW;                          // this wavefront's first channel
 
-    u32x4_a q[KS];
-    {
-        const uint16_t* qp = static_cast<const uint16_t*>(a.q) + (static_cast<size_t>(b) * rows + nc) * R + 8 * g;
-        static_for<KS>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-            q[i] = u32x4_a{0, 0, 0, 0};
-            if (i * 32 + 8 * g < R) q[i] = *reinterpret_cast<const u32x4_a*>(qp + i * 32);
-        });
-    }
-    const int limit = pos + nc / a.H + 1;            // keys this row may see: positions below it
-    const float scale2 = a.scale * kLog2e;
     const uint16_t* cb = static_cast<const uint16_t*>(a.c) + static_cast<size_t>(b) * a.capacity * R;
+    uint16_t* tile = tiles[wv];
 
     u32x4_a stage[LPT];
     auto fetch = [&](int64_t key0) {
         static_for<LPT>([&](auto I) {
             constexpr int i = decltype(I)::value;
-            const int u = i * NT + tid, tok = u / CH, ch = u % CH;
-            const int64_t key = key0 + tok < s1 ? key0 + tok : s1 - 1;       // rows past the slice: a copy, weight zero
-            stage[i] = u32x4_a{0, 0, 0, 0};
-            if (ch * 8 < R) stage[i] = *reinterpret_cast<const u32x4_a*>(cb + key * R + ch * 8);
+            const int u = i * kWave + lane, tok = u / CH, c = c0 + (u % CH) * 8;
+            // no branch around a load (it would be waited for at the join): rows past the slice are a copy with weight
+            // zero, columns past R a copy that meets zeros of q and whose output columns are never stored
+            const int64_t key = key0 + tok < s1 ? key0 + tok : s1 - 1;
+            stage[i] = *reinterpret_cast<const u32x4_a*>(cb + key * R + (c < R ? c : 0));
         });
     };
-    auto put = [&](int buf) {
-        static_for<LPT>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-            const int u = i * NT + tid, tok = u / CH, ch = u % CH;
-            *reinterpret_cast<u32x4_a*>(&tile[buf][tok * RP + ((ch ^ swz(tok)) * 8)]) = stage[i];
-        });
-    };
-    floatx4_a o[CT];
-    static_for<CT>([&](auto I) { o[decltype(I)::value] = floatx4_a{0, 0, 0, 0}; });
-    float m = kNone, l = 0.0f;
-    // element offsets inside a tile; pieces 16 apart (8 for the 64-wide rows) differ by a constant
-    constexpr int KLOW = KS < 4 ? KS : 4, VLOW = CT < 8 ? CT : 8;
-    int koff[KLOW], voff[VLOW];
-    static_for<KLOW>([&](auto I) { constexpr int i = decltype(I)::value; koff[i] = r16 * RP + (((i * 4 + g) ^ swz(r16)) * 8); });
-    {
-        const int row = 4 * g + (r16 >> 2);
-        static_for<VLOW>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-            voff[i] = row * RP + (((i * 2 + ((r16 & 3) >> 1)) ^ swz(row)) * 8) + (r16 & 1) * 4;
-        });
-    }
-
-    const int ntiles = static_cast<int>((s1 - s0 + kDecodeTile - 1) / kDecodeTile);
     fetch(s0);
-    put(0);
-    __syncthreads();
-    for (int it = 0; it < ntiles; it++) {
-        const int buf = it & 1;
-        if (it + 1 < ntiles) fetch(s0 + static_cast<int64_t>(it + 1) * kDecodeTile);
-        __builtin_amdgcn_sched_barrier(0);
-        const uint16_t* base = tile[buf];
-        floatx4_a s[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}};
+    __builtin_amdgcn_sched_barrier(0);
+    u32x4_a q[RT][KS];
+    int limit[RT];                                   // keys a row may see: positions below it
+    static_for<RT>([&](auto J) {
+        constexpr int j = decltype(J)::value;
+        const int n = n0 + j * 16 + r16 < rows ? n0 + j * 16 + r16 : rows - 1;
+        limit[j] = pos + n / a.H + 1;
+        const uint16_t* qp = static_cast<const uint16_t*>(a.q) + (static_cast<size_t>(b) * rows + n) * R;
         static_for<KS>([&](auto I) {
             constexpr int i = decltype(I)::value;
-            const uint16_t* p = base + koff[i % KLOW] + (i / KLOW) * 128;
-            s[0] = mma16<T>(*reinterpret_cast<const u32x4_a*>(p), q[i], s[0]);
-            s[1] = mma16<T>(*reinterpret_cast<const u32x4_a*>(p + 16 * RP), q[i], s[1]);
+            const int c = c0 + i * 32 + 8 * g;
+            const u32x4_a t = *reinterpret_cast<const u32x4_a*>(qp + (c < R ? c : 0));
+            q[j][i] = c < R ? t : u32x4_a{0, 0, 0, 0};
         });
-        // this lane: row n, tokens 4g + j and 16 + 4g + j of the tile
-        const int64_t key0 = s0 + static_cast<int64_t>(it) * kDecodeTile + 4 * g;
-        float p[8], mx = kNone;
-#pragma unroll
-        for (int u = 0; u < 2; u++)
-#pragma unroll
-            for (int j = 0; j < 4; j++) {
-                const int64_t key = key0 + 16 * u + j;
-                const float v = (key < limit && key < s1) ? s[u][j] * scale2 : -INFINITY;
-                p[4 * u + j] = v;
-                mx = fmaxf(mx, v);
-            }
-        mx = fmaxf(mx, __shfl_xor(mx, 16));
-        mx = fmaxf(mx, __shfl_xor(mx, 32));
-        if (__any(mx > m)) {
-            const float mn = fmaxf(m, mx), al = exp2_hw(m - mn);
-            l *= al;
-            static_for<CT>([&](auto I) {
-                constexpr int i = decltype(I)::value;
-#pragma unroll
-                for (int j = 0; j < 4; j++) o[i][j] *= al;
-            });
-            m = mn;
-        }
-#pragma unroll
-        for (int j = 0; j < 8; j++) { p[j] = exp2_hw(p[j] - m); l += p[j]; }
-        const u32x4_a pt = {pack2<T>(p[0], p[1]), pack2<T>(p[2], p[3]), pack2<T>(p[4], p[5]), pack2<T>(p[6], p[7])};
+    });
+    const int first_limit = pos + n0 / a.H + 1;      // the smallest of them: tiles below it need no mask
+    const float scale2 = a.scale * kLog2e;
+    auto put = [&]() {
+        static_for<LPT>([&](auto I) {
+            constexpr int i = decltype(I)::value;
+            const int u = i * kWave + lane, tok = u / CH, ch = u % CH;
+            *reinterpret_cast<u32x4_a*>(tile + tok * CW + ((ch ^ swz(tok)) * 8)) = stage[i];
+        });
+    };
+    floatx4_a o[RT][CT];
+    static_for<RT>([&](auto J) { static_for<CT>([&](auto I) { o[decltype(J)::value][decltype(I)::value] = floatx4_a{0, 0, 0, 0}; }); });
+    float m[RT], l[RT];
+    static_for<RT>([&](auto J) { m[decltype(J)::value] = kNone; l[decltype(J)::value] = 0.0f; });
+    int koff[KS], voff[CT];                          // elements inside the tile
+    static_for<KS>([&](auto I) { constexpr int i = decltype(I)::value; koff[i] = r16 * CW + (((i * 4 + g) ^ swz(r16)) * 8); });
+    {
+        const int row = 4 * g + (r16 >> 2);
         static_for<CT>([&](auto I) {
             constexpr int i = decltype(I)::value;
-            const uint16_t* vp = base + voff[i % VLOW] + (i / VLOW) * 128;
-            const short4_a v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)(vp));
-            const short4_a v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)(vp + 16 * RP));
-            const u32x2_a w0 = __builtin_bit_cast(u32x2_a, v0), w1 = __builtin_bit_cast(u32x2_a, v1);
-            o[i] = mma16<T>(u32x4_a{w0.x, w0.y, w1.x, w1.y}, pt, o[i]);
+            voff[i] = row * CW + (((i * 2 + ((r16 & 3) >> 1)) ^ swz(row)) * 8) + (r16 & 1) * 4;
         });
-        if (it + 1 < ntiles) put(buf ^ 1);           // its last readers passed the barrier of the previous iteration
-        __syncthreads();
     }
-    l += __shfl_xor(l, 16);
-    l += __shfl_xor(l, 32);
-    if (!valid) return;
-    if (g == 0) { ml[2 * n] = m; ml[2 * n + 1] = l; }
-    static_for<CT>([&](auto I) {
-        constexpr int i = decltype(I)::value;
-        const int ch = i * 16 + 4 * g;
-        if (ch < R) *reinterpret_cast<float4*>(acc + static_cast<size_t>(n) * R + ch) = make_float4(o[i][0], o[i][1], o[i][2], o[i][3]);
+    static_assert((16 / RPW) % CH == 0, "rows 16 apart are swizzled alike");
+
+    const int ntiles = static_cast<int>((s1 - s0 + kDecodeTile - 1) / kDecodeTile);
+    put();
+    for (int it = 0; it < ntiles; it++) {
+        if (it + 1 < ntiles) fetch(s0 + static_cast<int64_t>(it + 1) * kDecodeTile);
+        __builtin_amdgcn_sched_barrier(0);
+        u32x4_a k[2][KS];
+        static_for<KS>([&](auto I) {
+            constexpr int i = decltype(I)::value;
+            k[0][i] = *reinterpret_cast<const u32x4_a*>(tile + koff[i]);
+            k[1][i] = *reinterpret_cast<const u32x4_a*>(tile + koff[i] + 16 * CW);
+        });
+        floatx4_a s[RT][2];
+        static_for<RT>([&](auto J) { constexpr int j = decltype(J)::value; s[j][0] = s[j][1] = floatx4_a{0, 0, 0, 0}; });
+        static_for<KS>([&](auto I) {
+            constexpr int i = decltype(I)::value;
+            static_for<RT>([&](auto J) {
+                constexpr int j = decltype(J)::value;
+                s[j][0] = mma16<T>(k[0][i], q[j][i], s[j][0]);
+                s[j][1] = mma16<T>(k[1][i], q[j][i], s[j][1]);
+            });
+        });
+        // the second product's operands, ahead of the exchange
+        u32x4_a v[CT];
+        static_for<CT>([&](auto I) {
+            constexpr int i = decltype(I)::value;
+            const u32x2_a w0 = __builtin_bit_cast(u32x2_a, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)(tile + voff[i])));
+            const u32x2_a w1 = __builtin_bit_cast(u32x2_a, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)(tile + voff[i] + 16 * CW)));
+            v[i] = u32x4_a{w0.x, w0.y, w1.x, w1.y};
+        });
+        floatx4_a(*ex)[2 * RT][kWave] = exch[it & 1];
+        static_for<RT>([&](auto J) {
+            constexpr int j = decltype(J)::value;
+            ex[wv][2 * j][lane] = s[j][0];
+            ex[wv][2 * j + 1][lane] = s[j][1];
+        });
+        __syncthreads();     // (the other buffer's readers are done before they arrive here)
+        const int64_t tile0 = s0 + static_cast<int64_t>(it) * kDecodeTile, key0 = tile0 + 4 * g;
+        const bool whole = tile0 + kDecodeTile <= first_limit && tile0 + kDecodeTile <= s1;
+        static_for<RT>([&](auto J) {
+            constexpr int j = decltype(J)::value;
+            // this lane: row r16 of row tile j, keys key0 + jj and key0 + 16 + jj
+            float p[8], mx = kNone;
+#pragma unroll
+            for (int u = 0; u < 2; u++) {
+                floatx4_a t = ex[0][2 * j + u][lane];
+#pragma unroll
+                for (int w = 1; w < NW; w++) t += ex[w][2 * j + u][lane];
+#pragma unroll
+                for (int jj = 0; jj < 4; jj++) p[4 * u + jj] = t[jj] * scale2;
+            }
+            if (!whole) {
+#pragma unroll
+                for (int e = 0; e < 8; e++) {
+                    const int64_t key = key0 + 16 * (e >> 2) + (e & 3);
+                    if (key >= limit[j] || key >= s1) p[e] = -INFINITY;
+                }
+            }
+#pragma unroll
+            for (int e = 0; e < 8; e++) mx = fmaxf(mx, p[e]);
+            mx = fmaxf(mx, __shfl_xor(mx, 16));
+            mx = fmaxf(mx, __shfl_xor(mx, 32));
+            if (__any(mx > m[j])) {
+                const float mn = fmaxf(m[j], mx), al = exp2_hw(m[j] - mn);
+                l[j] *= al;
+                static_for<CT>([&](auto I) {
+                    constexpr int i = decltype(I)::value;
+                    o[j][i] *= al;
+                });
+                m[j] = mn;
+            }
+#pragma unroll
+            for (int e = 0; e < 8; e++) { p[e] = exp2_hw(p[e] - m[j]); l[j] += p[e]; }
+            const u32x4_a pt = {pack2<T>(p[0], p[1]), pack2<T>(p[2], p[3]), pack2<T>(p[4], p[5]), pack2<T>(p[6], p[7])};
+            static_for<CT>([&](auto I) {
+                constexpr int i = decltype(I)::value;
+                o[j][i] = mma16<T>(v[i], pt, o[j][i]);
+            });
+        });
+        if (it + 1 < ntiles) put();
+    }
+    static_for<RT>([&](auto J) {
+        constexpr int j = decltype(J)::value;
+        const int n = n0 + j * 16 + r16;
+        float ls = l[j] + __shfl_xor(l[j], 16);
+        ls += __shfl_xor(ls, 32);
+        if (n < rows) {
+            if (g == 0 && wv == 0) { ml[2 * n] = m[j]; ml[2 * n + 1] = ls; }
+            static_for<CT>([&](auto I) {
+                constexpr int i = decltype(I)::value;
+                const int c = c0 + i * 16 + 4 * g;
+                if (c < R) *reinterpret_cast<float4*>(acc + static_cast<size_t>(n) * R + c) = make_float4(o[j][i][0], o[j][i][1], o[j][i][2], o[j][i][3]);
+            });
+        }
     });
 }
 
-// grid (L * H, B), 128 threads: joins the slices of a row; the sink joins the denominator here, once.
+// grid (L * H, channel blocks of 64, B), 256 threads: joins the slices of a row; the sink joins the denominator here, once.
+// 16 lanes hold a block's channels, the 16 groups of them take the slices in turn.
 constexpr int kMaxSlices = 512;
 template <typename T>
-__global__ __launch_bounds__(128) void latent_merge_kernel(LatentDecodeArgs a) {
-    __shared__ float wgt[kMaxSlices], red[4];
-    const int n = blockIdx.x, b = blockIdx.y, rows = a.L * a.H, S = a.n_splits, R = a.R, tid = threadIdx.x;
+__global__ __launch_bounds__(256) void latent_merge_kernel(LatentDecodeArgs a) {
+    __shared__ float wgt[kMaxSlices], red[8];
+    __shared__ float4 sums[16][16];
+    const int n = blockIdx.x, b = blockIdx.z, rows = a.L * a.H, S = a.n_splits, R = a.R, tid = threadIdx.x;
+    const int ch = blockIdx.y * 64 + (tid & 15) * 4, grp = tid >> 4;
+    const int cc = ch < R ? ch : 0;
     const size_t first = static_cast<size_t>(b) * S * rows + n;
     const float sink2 = a.sink[n % a.H] * kLog2e;
-    float mx = sink2;
-    for (int s = tid; s < S; s += 128) mx = fmaxf(mx, a.workspace[2 * (first + static_cast<size_t>(s) * rows)]);
+    float mx = sink2, den = 0.0f;
+    for (int s = tid; s < S; s += 256) mx = fmaxf(mx, a.workspace[2 * (first + static_cast<size_t>(s) * rows)]);
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o));
     if ((tid & 63) == 0) red[tid >> 6] = mx;
     __syncthreads();
-    mx = fmaxf(red[0], red[1]);
-    float den = 0.0f;
-    for (int s = tid; s < S; s += 128) {
+    mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+    for (int s = tid; s < S; s += 256) {
         const float* p = a.workspace + 2 * (first + static_cast<size_t>(s) * rows);
         const float w = p[0] > kNone ? exp2_hw(p[0] - mx) : 0.0f;
         wgt[s] = w;
@@ -222,35 +271,36 @@ __global__ __launch_bounds__(128) void latent_merge_kernel(LatentDecodeArgs a) {
     }
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) den += __shfl_xor(den, o);
-    if ((tid & 63) == 0) red[2 + (tid >> 6)] = den;
+    if ((tid & 63) == 0) red[4 + (tid >> 6)] = den;
     __syncthreads();
-    const float inv = 1.0f / (red[2] + red[3] + exp2_hw(sink2 - mx));
-    const float* acc = a.workspace + pairs_floats(a) + first * R;
-    for (int ch = tid * 4; ch < R; ch += 512) {
-        float4 sum = make_float4(0, 0, 0, 0);
-        for (int s = 0; s < S; s++) {
-            const float w = wgt[s];
-            if (w == 0.0f) continue;                 // (an empty slice's accumulators were never written)
-            const float4 v = *reinterpret_cast<const float4*>(acc + static_cast<size_t>(s) * rows * R + ch);
-            sum.x = __builtin_fmaf(w, v.x, sum.x); sum.y = __builtin_fmaf(w, v.y, sum.y);
-            sum.z = __builtin_fmaf(w, v.z, sum.z); sum.w = __builtin_fmaf(w, v.w, sum.w);
-        }
-        *reinterpret_cast<uint2*>(static_cast<uint16_t*>(a.out) + (static_cast<size_t>(b) * rows + n) * R + ch) =
-            make_uint2(pack2<T>(sum.x * inv, sum.y * inv), pack2<T>(sum.z * inv, sum.w * inv));
+    const float* acc = a.workspace + pairs_floats(a) + first * R + cc;
+    float4 sum = make_float4(0, 0, 0, 0);
+#pragma unroll 4
+    for (int s = grp; s < S; s += 16) {
+        const float w = wgt[s];
+        const float4 v = *reinterpret_cast<const float4*>(acc + static_cast<size_t>(s) * rows * R);
+        const bool live = w != 0.0f;                 // (an empty slice's accumulators were never written)
+        sum.x = __builtin_fmaf(w, live ? v.x : 0.0f, sum.x); sum.y = __builtin_fmaf(w, live ? v.y : 0.0f, sum.y);
+        sum.z = __builtin_fmaf(w, live ? v.z : 0.0f, sum.z); sum.w = __builtin_fmaf(w, live ? v.w : 0.0f, sum.w);
     }
+    sums[grp][tid & 15] = sum;
+    __syncthreads();
+    if (grp != 0 || ch >= R) return;
+    for (int j = 1; j < 16; j++) {
+        const float4 v = sums[j][tid];
+        sum.x += v.x; sum.y += v.y; sum.z += v.z; sum.w += v.w;
+    }
+    const float inv = 1.0f / (red[4] + red[5] + red[6] + red[7] + exp2_hw(sink2 - mx));
+    *reinterpret_cast<uint2*>(static_cast<uint16_t*>(a.out) + (static_cast<size_t>(b) * rows + n) * R + ch) =
+        make_uint2(pack2<T>(sum.x * inv, sum.y * inv), pack2<T>(sum.z * inv, sum.w * inv));
 }
 
 int launch_latent_decode(const LatentDecodeArgs& a, int dtype, hipStream_t st) {
     const int rows = a.L * a.H;
-    // (a single wavefront's share of a 512-wide tile in flight does not fit its registers beside the accumulators)
-    const int rw = rows <= 16 && a.R <= 256 ? 1 : rows <= 32 ? 2 : 4;
-    dim3 grid(a.n_splits, (rows + 16 * rw - 1) / (16 * rw), a.B), block(kWave * rw);
-#define PQ_LD(T, RP)                                                                                                 \
-    do {                                                                                                             \
-        if (rw == 1 && RP <= 256) hipLaunchKernelGGL((latent_decode_kernel<T, (RP <= 256 ? RP : 256), 1>), grid, block, 0, st, a);                    \
-        else if (rw == 2) hipLaunchKernelGGL((latent_decode_kernel<T, RP, 2>), grid, block, 0, st, a);               \
-        else hipLaunchKernelGGL((latent_decode_kernel<T, RP, 4>), grid, block, 0, st, a);                            \
-    } while (0)
+    const int rt = rows <= 16 ? 1 : rows <= 32 ? 2 : 4;
+    dim3 grid(a.n_splits, (rows + 16 * rt - 1) / (16 * rt), a.B);
+#define PQ_LD1(T, RP, RT) hipLaunchKernelGGL((latent_decode_kernel<T, RP, RT>), grid, dim3(kWave * DecodeShape<RP>::NW), 0, st, a)
+#define PQ_LD(T, RP) do { if (rt == 1) PQ_LD1(T, RP, 1); else if (rt == 2) PQ_LD1(T, RP, 2); else PQ_LD1(T, RP, 4); } while (0)
 #define PQ_LDT(T)                                                                                                    \
     do {                                                                                                             \
         if (a.R <= 64) PQ_LD(T, 64); else if (a.R <= 128) PQ_LD(T, 128);                                             \
@@ -259,9 +309,10 @@ int launch_latent_decode(const LatentDecodeArgs& a, int dtype, hipStream_t st) {
     if (dtype == 0) PQ_LDT(F16); else PQ_LDT(BF16);
 #undef PQ_LDT
 #undef PQ_LD
+#undef PQ_LD1
     int err = static_cast<int>(hipGetLastError());
     if (err) return err;
-    dim3 mgrid(rows, a.B), mblock(128);
+    dim3 mgrid(rows, (a.R + 63) / 64, a.B), mblock(256);
     if (dtype == 0) hipLaunchKernelGGL(latent_merge_kernel<F16>, mgrid, mblock, 0, st, a);
     else hipLaunchKernelGGL(latent_merge_kernel<BF16>, mgrid, mblock, 0, st, a);
     return static_cast<int>(hipGetLastError());
@@ -362,11 +413,12 @@ __global__ __launch_bounds__(256, DKP <= 128 ? 2 : 1) void latent_prefill_kernel
 
     u32x4_a q[KS];
     {
-        const uint16_t* qp = static_cast<const uint16_t*>(a.q) + ((static_cast<size_t>(b) * a.L + qc) * H + h) * D + 8 * hi;
+        const uint16_t* qp = static_cast<const uint16_t*>(a.q) + ((static_cast<size_t>(b) * a.L + qc) * H + h) * D;
         static_for<KS>([&](auto I) {
             constexpr int i = decltype(I)::value;
-            q[i] = u32x4_a{0, 0, 0, 0};
-            if (i * 16 + 8 * hi < D) q[i] = *reinterpret_cast<const u32x4_a*>(qp + i * 16);
+            const int c = i * 16 + 8 * hi;
+            const u32x4_a t = *reinterpret_cast<const u32x4_a*>(qp + (c < D ? c : 0));
+            q[i] = c < D ? t : u32x4_a{0, 0, 0, 0};
         });
     }
     const uint16_t* kb = static_cast<const uint16_t*>(a.k) + (static_cast<size_t>(b) * a.Lk * H + h) * D;
@@ -377,15 +429,15 @@ __global__ __launch_bounds__(256, DKP <= 128 ? 2 : 1) void latent_prefill_kernel
             constexpr int i = decltype(I)::value;
             const int u = i * 256 + tid, tok = u / (DKP / 8), ch = u % (DKP / 8);
             int key = it * kPrefillKeys + tok;
-            key = key < a.Lk ? key : a.Lk - 1;                      // keys past the end: a copy, weight zero
-            ks[i] = u32x4_a{0, 0, 0, 0};
-            if (ch * 8 < D) ks[i] = *reinterpret_cast<const u32x4_a*>(kb + static_cast<size_t>(key) * H * D + ch * 8);
+            // no branch around a load (it would be waited for at the join): keys past the end are a copy with weight zero,
+            // columns past D a copy that meets zeros of q
+            key = key < a.Lk ? key : a.Lk - 1;
+            ks[i] = *reinterpret_cast<const u32x4_a*>(kb + static_cast<size_t>(key) * H * D + (ch * 8 < D ? ch * 8 : 0));
         });
         static_for<VLOADS>([&](auto I) {
             constexpr int i = decltype(I)::value;
-            const int u = i * 256 + tid, ch = u / 8, piece = u % 8;
-            vs[i] = u32x4_a{0, 0, 0, 0};
-            if (ch < Dv) vs[i] = *reinterpret_cast<const u32x4_a*>(vb + static_cast<size_t>(ch) * a.ldv + it * kPrefillKeys + piece * 8);
+            const int u = i * 256 + tid, piece = u % 8, ch = u / 8 < Dv ? u / 8 : Dv - 1;      // (rows past Dv are never stored)
+            vs[i] = *reinterpret_cast<const u32x4_a*>(vb + static_cast<size_t>(ch) * a.ldv + it * kPrefillKeys + piece * 8);
         });
     };
     auto put = [&](int buf) {

@@ -117,10 +117,11 @@ int pq_head_linear(const void* x, int64_t x_row_stride, int64_t x_head_stride, c
 int pq_latent_decode_plan(int B, int L, int H, int64_t max_keys, int n_cus) {
     if (B < 1 || L < 1 || H < 1 || max_keys < 1) return 1;
     if (n_cus <= 0) n_cus = 256;
-    const int64_t rows = static_cast<int64_t>(L) * H, per = rows <= 32 ? 32 : 64;
+    const int64_t rows = static_cast<int64_t>(L) * H, per = rows <= 16 ? 16 : rows <= 32 ? 32 : 64;
     const int64_t groups = static_cast<int64_t>(B) * ((rows + per - 1) / per);
-    // one workgroup per compute unit; every slice costs a partial of R floats per row, so a slice keeps at least 128 keys
-    int64_t n = (n_cus + groups - 1) / groups, most = (max_keys + 127) / 128;
+    // what the compute units hold at once (two workgroups of up to 32 rows, one of 64); every slice costs a partial of R
+    // floats per row, so a slice keeps at least 128 keys
+    int64_t n = (n_cus * (per <= 32 ? 2 : 1) + groups - 1) / groups, most = (max_keys + 127) / 128;
     n = n < most ? n : most;
     return static_cast<int>(n < 1 ? 1 : n > 512 ? 512 : n);
 }

@@ -88,11 +88,11 @@ def test_norm_conv_left_padding(gpu):
 @pytest.mark.parametrize("q_rank,kv_rank,extra", [(64, 96, 128), (18, 36, 5), (11, 13, 0), (1536, 512, 64), (7, 1, 3)])
 def test_latent_norm(gpu, q_rank, kv_rank, extra):
     g = torch.Generator().manual_seed(q_rank)
-    for dt in DT:
-        B, L, pos = 3, 5, 9
+    for dt, L in [(dt, L) for dt in DT for L in (5, 401)]:        # few tokens: a workgroup each, many: a wavefront each
+        B, pos = 3, 9
         p = rand(g, B, L, q_rank + kv_rank + extra, dt=dt, s=2.0)
         wq, wc = (1 + rand(g, q_rank, s=0.3)).to(DT[dt]), (1 + rand(g, kv_rank, s=0.3)).to(DT[dt])
-        cache = torch.full((B, 20, kv_rank), 7.0, dtype=DT[dt], device=gpu)
+        cache = torch.full((B, L + 15, kv_rank), 7.0, dtype=DT[dt], device=gpu)
         cq = ops.latent_norm(p.to(gpu), wq.to(gpu), wc.to(gpu), cache, 1e-3, pos)
         assert err(cq, do.rms_norm(p[..., :q_rank].double(), wq.double(), 1e-3)) < TOL[dt]
         assert err(cache[:, pos:pos + L], do.rms_norm(p[..., q_rank:q_rank + kv_rank].double(), wc.double(), 1e-3)) < TOL[dt]
