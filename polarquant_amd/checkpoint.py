@@ -91,6 +91,7 @@ def load_state(model: torch.nn.Module, shard_files: Iterable[str], dtype: torch.
     from safetensors import safe_open
     params = _named_tensors(model)
     tied = getattr(model.config, "tie_word_embeddings", False)
+    unused = model.unused_tensors() if hasattr(model, "unused_tensors") else ()
     seen = set()
     with torch.no_grad():
         for fn in shard_files:
@@ -99,6 +100,8 @@ def load_state(model: torch.nn.Module, shard_files: Iterable[str], dtype: torch.
                     if name.endswith("rotary_emb.inv_freq"):
                         continue
                     if name == "lm_head.weight" and tied:
+                        continue
+                    if name in unused:
                         continue
                     if name not in params:
                         raise KeyError("polarquant_amd: %s holds %r, which the model has no parameter for" % (fn, name))

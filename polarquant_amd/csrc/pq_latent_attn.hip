@@ -77,13 +77,11 @@ __global__ __launch_bounds__(kWave * DecodeShape<RP>::NW, RT <= 2 ? 2 : 1) void 
     const int tid = threadIdx.x, lane = tid & 63, wv = tid / kWave, r16 = lane & 15, g = lane >> 4;
     const int b = blockIdx.z, split = blockIdx.x, R = a.R, rows = a.L * a.H, n0 = blockIdx.y * 16 * RT;
     const int pos = a.pos_dev ? *a.pos_dev : a.pos;
-    int64_t total = static_cast<int64_t>(pos) + a.L;
-    if (total > a.capacity) total = a.capacity;
+    const int total = static_cast<int>(static_cast<int64_t>(pos) + a.L < a.capacity ? pos + a.L : a.capacity);   // (below 2^30)
     const int lo = a.start ? a.start[b] : 0;
-    const int len = static_cast<int>(total) - lo;
-    const int per = ((len + a.n_splits - 1) / a.n_splits + kDecodeTile - 1) / kDecodeTile * kDecodeTile;
-    const int64_t s0 = lo + static_cast<int64_t>(split) * per;
-    const int64_t s1 = s0 + per < total ? s0 + per : total;
+    const int per = ((total - lo + a.n_splits - 1) / a.n_splits + kDecodeTile - 1) / kDecodeTile * kDecodeTile;
+    const int64_t begin = lo + static_cast<int64_t>(split) * per;
+    const int s0 = static_cast<int>(begin < total ? begin : total), s1 = begin + per < total ? s0 + per : total;
     const size_t part = (static_cast<size_t>(b) * a.n_splits + split) * rows;
     float* ml = a.workspace + 2 * part;
     float* acc = a.workspace + pairs_floats(a) + part * R;
@@ -98,14 +96,22 @@ __global__ __launch_bounds__(kWave * DecodeShape<RP>::NW, RT <= 2 ? 2 : 1) void 
     uint16_t* tile = tiles[wv];
 
     u32x4_a stage[LPT];
-    auto fetch = [&](int64_t key0) {
+    uint32_t off[LPT], col[LPT];                     // elements from the tile's first key
+    static_for<LPT>([&](auto I) {
+        constexpr int i = decltype(I)::value;
+        const int u = i * kWave + lane, c = c0 + (u % CH) * 8;
+        col[i] = c < R ? c : 0;
+        off[i] = static_cast<uint32_t>(u / CH) * R + col[i];
+    });
+    auto fetch = [&](int key0) {
+        const uint16_t* base = cb + static_cast<int64_t>(key0) * R;
+        const int last = s1 - 1 - key0;              // uniform
         static_for<LPT>([&](auto I) {
             constexpr int i = decltype(I)::value;
-            const int u = i * kWave + lane, tok = u / CH, c = c0 + (u % CH) * 8;
             // no branch around a load (it would be waited for at the join): rows past the slice are a copy with weight
             // zero, columns past R a copy that meets zeros of q and whose output columns are never stored
-            const int64_t key = key0 + tok < s1 ? key0 + tok : s1 - 1;
-            stage[i] = *reinterpret_cast<const u32x4_a*>(cb + key * R + (c < R ? c : 0));
+            const int tok = (i * kWave + lane) / CH;
+            stage[i] = *reinterpret_cast<const u32x4_a*>(base + (tok <= last ? off[i] : static_cast<uint32_t>(last) * R + col[i]));
         });
     };
     fetch(s0);
@@ -148,10 +154,10 @@ __global__ __launch_bounds__(kWave * DecodeShape<RP>::NW, RT <= 2 ? 2 : 1) void 
     }
     static_assert((16 / RPW) % CH == 0, "rows 16 apart are swizzled alike");
 
-    const int ntiles = static_cast<int>((s1 - s0 + kDecodeTile - 1) / kDecodeTile);
+    const int ntiles = (s1 - s0 + kDecodeTile - 1) / kDecodeTile;
     put();
     for (int it = 0; it < ntiles; it++) {
-        if (it + 1 < ntiles) fetch(s0 + static_cast<int64_t>(it + 1) * kDecodeTile);
+        if (it + 1 < ntiles) fetch(s0 + (it + 1) * kDecodeTile);
         __builtin_amdgcn_sched_barrier(0);
         u32x4_a k[2][KS];
         static_for<KS>([&](auto I) {
@@ -184,7 +190,7 @@ __global__ __launch_bounds__(kWave * DecodeShape<RP>::NW, RT <= 2 ? 2 : 1) void 
             ex[wv][2 * j + 1][lane] = s[j][1];
         });
         __syncthreads();     // (the other buffer's readers are done before they arrive here)
-        const int64_t tile0 = s0 + static_cast<int64_t>(it) * kDecodeTile, key0 = tile0 + 4 * g;
+        const int tile0 = s0 + it * kDecodeTile, key0 = tile0 + 4 * g;
         const bool whole = tile0 + kDecodeTile <= first_limit && tile0 + kDecodeTile <= s1;
         static_for<RT>([&](auto J) {
             constexpr int j = decltype(J)::value;
@@ -201,7 +207,7 @@ __global__ __launch_bounds__(kWave * DecodeShape<RP>::NW, RT <= 2 ? 2 : 1) void 
             if (!whole) {
 #pragma unroll
                 for (int e = 0; e < 8; e++) {
-                    const int64_t key = key0 + 16 * (e >> 2) + (e & 3);
+                    const int key = key0 + 16 * (e >> 2) + (e & 3);
                     if (key >= limit[j] || key >= s1) p[e] = -INFINITY;
                 }
             }
@@ -424,15 +430,16 @@ __global__ __launch_bounds__(256, DKP <= 128 ? 2 : 1) void latent_prefill_kernel
     const uint16_t* kb = static_cast<const uint16_t*>(a.k) + (static_cast<size_t>(b) * a.Lk * H + h) * D;
     const uint16_t* vb = static_cast<const uint16_t*>(a.vt) + (static_cast<size_t>(b) * H + h) * Dv * a.ldv;
     u32x4_a ks[KLOADS], vs[VLOADS];
+    const uint32_t k_row = static_cast<uint32_t>(H) * D;
     auto fetch = [&](int it) {
+        const uint16_t* kbase = kb + static_cast<size_t>(it) * kPrefillKeys * k_row;
+        const int last = a.Lk - 1 - it * kPrefillKeys;             // uniform
         static_for<KLOADS>([&](auto I) {
             constexpr int i = decltype(I)::value;
             const int u = i * 256 + tid, tok = u / (DKP / 8), ch = u % (DKP / 8);
-            int key = it * kPrefillKeys + tok;
             // no branch around a load (it would be waited for at the join): keys past the end are a copy with weight zero,
             // columns past D a copy that meets zeros of q
-            key = key < a.Lk ? key : a.Lk - 1;
-            ks[i] = *reinterpret_cast<const u32x4_a*>(kb + static_cast<size_t>(key) * H * D + (ch * 8 < D ? ch * 8 : 0));
+            ks[i] = *reinterpret_cast<const u32x4_a*>(kbase + (static_cast<uint32_t>(tok <= last ? tok : last) * k_row + (ch * 8 < D ? ch * 8 : 0)));
         });
         static_for<VLOADS>([&](auto I) {
             constexpr int i = decltype(I)::value;

@@ -138,7 +138,7 @@ int pq_validate_latent_decode(const void* q, const void* c, int64_t capacity, co
     if (!q || !c || !sink || !out) return PQ_ERR_NULL_POINTER;
     if (!any_dtype(dtype)) return PQ_ERR_BAD_DTYPE;
     if (int rc = check_tokens(B, L)) return rc;
-    if (H < 1 || R < 1 || R > 7168 || static_cast<int64_t>(L) * H > (1 << 24) || pos < 0) return PQ_ERR_BAD_SHAPE;
+    if (H < 1 || H > 65535 || R < 1 || R > 7168 || static_cast<int64_t>(L) * H > (1 << 24) || pos < 0) return PQ_ERR_BAD_SHAPE;
     if (capacity < 1 || capacity > kMaxTokens || static_cast<int64_t>(pos) + L > capacity) return PQ_ERR_BAD_STRIDE;
     if (!aligned(q, 16) || !aligned(c, 16) || !aligned(out, 16) || !aligned(sink, 4) || (start && !aligned(start, 4)) ||
         (pos_dev && !aligned(pos_dev, 4)))
@@ -169,7 +169,7 @@ int pq_validate_latent_prefill(const void* q, const void* k, const void* vt, int
     if (!q || !k || !vt || !sink || !out) return PQ_ERR_NULL_POINTER;
     if (dtype != PQ_F16 && dtype != PQ_BF16) return PQ_ERR_BAD_DTYPE;
     if (int rc = check_tokens(B, L)) return rc;
-    if (H < 1 || !pq_latent_prefill_takes(D, Dv, dtype) || Lk < L || Lk > kMaxTokens || (L + 127) / 128 > 65535) return PQ_ERR_BAD_SHAPE;
+    if (H < 1 || H > 65535 || !pq_latent_prefill_takes(D, Dv, dtype) || Lk < L || Lk > kMaxTokens || (L + 127) / 128 > 65535) return PQ_ERR_BAD_SHAPE;
     if (vt_row_stride % 64 || vt_row_stride < Lk || (gate && gate_row_stride < static_cast<int64_t>(H) * Dv)) return PQ_ERR_BAD_STRIDE;
     if (!aligned(q, 16) || !aligned(k, 16) || !aligned(vt, 16) || !aligned(out, 8) || (gate && !aligned(gate, 8)) || !aligned(sink, 4) ||
         (start && !aligned(start, 4)))

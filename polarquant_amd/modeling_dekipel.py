@@ -108,3 +108,7 @@ class DekipelForCausalLM(LatentForCausalLM):
             if layer.mlp is not None:
                 out[l + "mlp.up"], out[l + "mlp.down"] = layer.mlp.up, layer.mlp.down
         return out
+
+    def unused_tensors(self):
+        """Names a checkpoint may hold that nothing reads: the norms and convolution of a feed-forward that a layer does not have."""
+        return {"l%d.%s" % (i, n) for i, layer in enumerate(self.model.layers) if layer.mlp is None for n in ("norm2", "norm2b", "canon2")}

@@ -65,7 +65,7 @@ def main(argv=None) -> int:
         family = family_of(json.load(f))
     if family.polar_cache:
         print("trace_run: %s models run in half precision on whole prompts only" % family.name, file=sys.stderr)
-        return 3
+        return 2
     build.ensure(family.libraries, verbose=False)
     torch.backends.cuda.matmul.allow_tf32 = False
     torch.backends.cuda.matmul.allow_bf16_reduced_precision_reduction = False

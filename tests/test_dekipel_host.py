@@ -108,6 +108,12 @@ def test_checkpoint_must_hold_every_tensor(tmp_path):
         ck.load_pretrained(str(tmp_path / "b"), torch.bfloat16, "cpu")
 
 
+def test_a_layer_without_feed_forward_ignores_its_norms(tmp_path):
+    w = do.random_weights(dc.EVEN, 2)
+    dc.write(str(tmp_path), dc.EVEN, 0, weights=dict(w, **{"l1.norm2": torch.ones(192), "l1.canon2": torch.ones(192, 3)}))
+    assert "l1.norm2" not in ck.load_pretrained(str(tmp_path), torch.bfloat16, "cpu").checkpoint_tensors()
+
+
 def test_left_padding_of_a_mask():
     pad = LatentModel._left_padding
     assert pad(None) is None and pad(torch.ones(2, 5)) is None
