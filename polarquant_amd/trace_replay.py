@@ -1,12 +1,14 @@
-"""Replay of given token ids through a model (bin/trace_run).
+"""Replay of recorded token ids through a model (bin/trace_run), for comparing logits between builds, dtypes and ways of
+cutting a sequence.
 
-Standard input holds one JSON object per line:
+Steps come as JSON lines on standard input: `step` (a number), `entries` (per request: `id`, the next `tokens`, and `want`,
+indices into them) and `end` (ids that are done).  For example
 
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+    {"step": 7, "entries": [{"id": "chat-1", "tokens": [101, 9], "want": [1]}], "end": ["chat-1"]}
 
-Each entry's tokens run through the model's forward on the cache that the request's earlier steps left; the logits at the
-places `want` names go to <out>/<step>.f32 (little-endian float32, [wanted, vocab], in the order of the entries), then
-"done <step>" is printed.  Requests in `end` give their cache back; its memory serves later requests.  Nothing is sampled.
+A request's tokens continue from the cache its earlier steps left.  Wanted logits go to <out>/<step>.f32 as rows of
+little-endian float32, entry by entry; each finished step is acknowledged by a line "done <step>".  An ended request's cache
+memory is used again by later requests.
 """
 from __future__ import annotations
 

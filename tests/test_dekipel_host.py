@@ -190,11 +190,11 @@ def test_decode_arguments_and_plan(lib):
 
 def test_prefill_arguments(lib):
     def call(**kw):
-        d = dict(q=A, k=A, vt=A, ld=128, sink=A, g=None, gr=0, start=None, out=A, B=1, L=20, Lk=100, H=3, D=64, Dv=48, dt=0)
+        d = dict(q=A, k=A, vt=A, ld=128, sink=A, g=None, gr=0, start=None, out=A, B=1, L=20, Lk=100, H=3, D=64, Dv=40, dt=0)
         d.update(kw)
         return lib.pq_validate_latent_prefill(*[d[k] for k in ("q", "k", "vt", "ld", "sink", "g", "gr", "start", "out", "B", "L", "Lk", "H", "D", "Dv", "dt")])
     assert call() == OK and call(ld=100) == STRIDE and call(ld=64) == STRIDE and call(Lk=19) == SHAPE and call(dt=2) == DTYPE
-    assert call(D=20) == SHAPE and call(D=264) == SHAPE and call(Dv=257) == SHAPE and call(g=A, gr=143) == STRIDE and call(g=A, gr=144) == OK
+    assert call(D=20) == SHAPE and call(D=264) == SHAPE and call(Dv=257) == SHAPE and call(g=A, gr=119) == STRIDE and call(g=A, gr=120) == OK
     assert lib.pq_latent_prefill_takes(192, 128, 1) == 1 and lib.pq_latent_prefill_takes(192, 128, 2) == 0
 
 
