@@ -13,7 +13,7 @@ from ctypes import c_char_p, c_float, c_int, c_int64, c_size_t, c_uint, c_void_p
 HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(HERE, "libpolarquant_hip.so")
 
-PQ_F16, PQ_BF16, PQ_F32 = 0, 1, 2          # float32: the latent-attention entry points only
+PQ_F16, PQ_BF16, PQ_F32 = 0, 1, 2          # float32: not in the polar-key library
 PQ_EPI_PLAIN, PQ_EPI_RELU_SQ, PQ_EPI_SIGMOID_GATE, PQ_EPI_F32 = 0, 1, 2, 3
 PQ_WRAP_FP32 = 1
 PQ_ANGLE_UNIFORM = 2
@@ -94,17 +94,25 @@ BENCH_SIGNATURES = {
 }
 
 
-# latent attention and the layer steps around it (include/polarquant_latent.h): a library of their own, so that a decoder
-# that needs nothing else need not build the polar-key kernels
-LATENT_LIB_PATH = os.path.join(HERE, "libpolarquant_latent.so")
-LATENT_SIGNATURES = {
+# the steps between mixers and matrix products (include/polarquant_steps.h) and the mixers' kernels, by family
+# (include/polarquant_latent.h): libraries of their own, so that a decoder builds only what it runs
+STEPS_LIB_PATH = os.path.join(HERE, "libpolarquant_steps.so")
+STEPS_SIGNATURES = {
     "pq_norm_conv": (c_int, [c_void_p] * 11 + [c_int] * 6 + [c_float] + [c_int] + [c_void_p]),
     "pq_validate_norm_conv": (c_int, [c_void_p] * 11 + [c_int] * 7),
-    "pq_latent_norm": (c_int, [c_void_p] + [c_int64] + [c_void_p] * 4 + [c_int64] + [c_void_p] + [c_int] * 5 + [c_float] + [c_int] + [c_void_p]),
-    "pq_validate_latent_norm": (c_int, [c_void_p] + [c_int64] + [c_void_p] * 4 + [c_int64] + [c_void_p] + [c_int] * 6),
     "pq_relu_sq": (c_int, [c_void_p] * 2 + [c_size_t] + [c_int] + [c_void_p]),
+    "pq_gelu_mul": (c_int, [c_void_p] * 2 + [c_int64, c_void_p, c_int64, c_int64, c_int, c_int, c_void_p]),
+    "pq_stream_add": (c_int, [c_void_p] * 5 + [c_int64, c_int, c_int, c_void_p]),
+    "pq_embed_rows": (c_int, [c_void_p] * 2 + [c_float, c_void_p, c_int64, c_int, c_int64, c_int, c_void_p]),
+    "pq_softcap": (c_int, [c_void_p, c_size_t, c_float, c_float, c_void_p]),
     "pq_head_linear": (c_int, [c_void_p] + [c_int64] * 2 + [c_void_p] * 2 + [c_int64] + [c_void_p] + [c_int64] * 2 + [c_int] * 6 + [c_void_p]),
     "pq_validate_head_linear": (c_int, [c_void_p] + [c_int64] * 2 + [c_void_p] * 2 + [c_int64] + [c_void_p] + [c_int64] * 2 + [c_int] * 6),
+}
+
+LATENT_LIB_PATH = os.path.join(HERE, "libpolarquant_latent.so")
+LATENT_SIGNATURES = {
+    "pq_latent_norm": (c_int, [c_void_p] + [c_int64] + [c_void_p] * 4 + [c_int64] + [c_void_p] + [c_int] * 5 + [c_float] + [c_int] + [c_void_p]),
+    "pq_validate_latent_norm": (c_int, [c_void_p] + [c_int64] + [c_void_p] * 4 + [c_int64] + [c_void_p] + [c_int] * 6),
     "pq_latent_decode_plan": (c_int, [c_int] * 3 + [c_int64] + [c_int]),
     "pq_latent_decode_workspace_bytes": (c_size_t, [c_int] * 5),
     "pq_latent_decode": (c_int, [c_void_p] * 2 + [c_int64] + [c_void_p] * 3 + [c_int] + [c_void_p] + [c_int] * 4 + [c_float] + [c_int] + [c_void_p] + [c_size_t] + [c_int] + [c_void_p]),
@@ -112,6 +120,27 @@ LATENT_SIGNATURES = {
     "pq_latent_prefill_takes": (c_int, [c_int] * 3),
     "pq_latent_prefill": (c_int, [c_void_p] * 3 + [c_int64] + [c_void_p] * 2 + [c_int64] + [c_void_p] * 2 + [c_int] * 6 + [c_float] + [c_int] + [c_void_p]),
     "pq_validate_latent_prefill": (c_int, [c_void_p] * 3 + [c_int64] + [c_void_p] * 2 + [c_int64] + [c_void_p] * 2 + [c_int] * 7),
+}
+
+
+# windowed attention and recurrent mixers (include/polarquant_recurrent.h)
+RECURRENT_LIB_PATH = os.path.join(HERE, "libpolarquant_recurrent.so")
+RECURRENT_SIGNATURES = {
+    "pq_qk_norm": (c_int, [c_void_p] * 3 + [c_int64] + [c_void_p] * 7 + [c_int] * 8 + [c_float, c_int, c_void_p]),
+    "pq_ring_append": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p] + [c_int] * 8 + [c_void_p]),
+    "pq_window_plan": (c_int, [c_int] * 6),
+    "pq_window_workspace_bytes": (c_size_t, [c_int] * 5),
+    "pq_validate_window_attn": (c_int, [c_void_p] * 4 + [c_int64, c_void_p, c_int64] + [c_void_p] * 3 + [c_int, c_void_p, c_int64]
+                                + [c_int] * 9 + [c_void_p, c_size_t, c_int]),
+    "pq_window_attn": (c_int, [c_void_p] * 4 + [c_int64, c_void_p, c_int64] + [c_void_p] * 3 + [c_int, c_void_p, c_int64] + [c_int] * 8
+                       + [c_float, c_float, c_int, c_void_p, c_size_t, c_int, c_void_p]),
+    "pq_validate_delta_prep": (c_int, [c_int] * 7 + [c_void_p, c_void_p, c_int64, c_int64, c_int]),
+    "pq_delta_prep": (c_int, [c_void_p] * 4 + [c_int64, c_void_p, c_int64] + [c_void_p] * 16 + [c_int] * 9 + [c_void_p]),
+    "pq_delta_scan": (c_int, [c_void_p] * 11 + [c_int] * 8 + [c_void_p]),
+    "pq_memory_gates": (c_int, [c_void_p, c_void_p, c_int64] + [c_void_p] * 4 + [c_int64, c_int, c_float, c_int, c_void_p]),
+    "pq_memory_scan": (c_int, [c_void_p] * 3 + [c_int64] + [c_void_p] * 6 + [c_float, c_void_p, c_void_p] + [c_int] * 7 + [c_void_p]),
+    "pq_head_norm_gate": (c_int, [c_void_p] * 3 + [c_int, c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_int, c_float, c_float, c_int,
+                                  c_void_p]),
 }
 
 
@@ -150,9 +179,19 @@ def lib() -> ctypes.CDLL:
     return _load(LIB_PATH, SIGNATURES)
 
 
+def steps_lib() -> ctypes.CDLL:
+    """The layer steps' library."""
+    return _load(STEPS_LIB_PATH, STEPS_SIGNATURES)
+
+
 def latent_lib() -> ctypes.CDLL:
     """The latent-attention library."""
     return _load(LATENT_LIB_PATH, LATENT_SIGNATURES)
+
+
+def recurrent_lib() -> ctypes.CDLL:
+    """The library of windowed attention and recurrent mixers."""
+    return _load(RECURRENT_LIB_PATH, RECURRENT_SIGNATURES)
 
 
 def bench_lib() -> ctypes.CDLL:

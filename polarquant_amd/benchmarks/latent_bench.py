@@ -179,7 +179,7 @@ def _throughput(name, model, decoder, B, L, new, layers):
 
 
 def models(s, B, L, emit, layers=4, new=64, which=("dekipel", "llama_polar")):
-    from ..graph_decode import LatentGraphDecoder, PolarGraphDecoder
+    from ..graph_decode import LayeredGraphDecoder, PolarGraphDecoder
     from ..modeling_common import PolarConfig
     from .e2e_bench import build_model
     dev = torch.device("cuda:0")
@@ -188,7 +188,7 @@ def models(s, B, L, emit, layers=4, new=64, which=("dekipel", "llama_polar")):
         if "dekipel" in which:
             torch.cuda.reset_peak_memory_stats()
             m = build_dekipel(s, layers, dev)
-            out["dekipel"] = _throughput("dekipel", m, LatentGraphDecoder(m, L + new + 128), B, L, new, layers)
+            out["dekipel"] = _throughput("dekipel", m, LayeredGraphDecoder(m, L + new + 128), B, L, new, layers)
             emit(out["dekipel"])
             del m
             torch.cuda.empty_cache()

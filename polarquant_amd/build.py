@@ -1,7 +1,7 @@
 """Build recipe of the HIP library: hipcc for gfx950, in-tree.
 
     python -m polarquant_amd.build                    # (re)build polarquant_amd/libpolarquant_hip.so, its test build and libpolarquant_bench.so
-    python -m polarquant_amd.build --latent           # libpolarquant_latent.so alone
+    python -m polarquant_amd.build --layers [steps] [latent] [recurrent]   # those libraries alone
     python -m polarquant_amd.build --phase-timers     # the measuring build (benchmarks/phase_timing.py)
     python -m polarquant_amd.build --probe no_values  # a probe build (benchmarks/probe_bench.py)
 
@@ -28,9 +28,14 @@ UNITS = [("pq_attn.hip", ("PQ_DTYPE=0",), ".f16"), ("pq_attn.hip", ("PQ_DTYPE=1"
          ("pq_scores.hip", (), ""), ("pq_quantize.hip", (), ""), ("pq_linear.hip", (), ""), ("pq_attn_common.hip", (), ""),
          ("pq_capi.hip", (), ""), ("pq_values.hip", (), ""), ("pq_decode_ops.hip", (), "")]
 SOURCES = sorted({u[0] for u in UNITS})
-# latent attention and the layer steps around it: a library of their own, all a Dekipel model needs
-LATENT_LIB = os.path.join(HERE, "libpolarquant_latent.so")
-LATENT_UNITS = [("pq_latent.hip", (), ""), ("pq_latent_attn.hip", (), ""), ("pq_head_linear.hip", (), ""), ("pq_latent_capi.hip", (), "")]
+# libraries of their own, so that a model builds only what it runs: the steps between mixers and matrix products, and the
+# kernels of the mixers by family
+LAYER_UNITS = {
+    "steps": [("pq_steps.hip", (), ""), ("pq_head_linear.hip", (), ""), ("pq_steps_capi.hip", (), "")],
+    "latent": [("pq_latent_attn.hip", (), ""), ("pq_latent_norm.hip", (), ""), ("pq_latent_capi.hip", (), "")],
+    "recurrent": [("pq_window_attn.hip", (), ""), ("pq_recurrent.hip", (), ""), ("pq_recurrent_capi.hip", (), "")],
+}
+LAYER_LIBS = {name: os.path.join(HERE, "libpolarquant_%s.so" % name) for name in LAYER_UNITS}
 # measurement aids (a plain streaming read, the attention kernel's loads without its arithmetic): a library of
 # their own, loaded by bench.py and its tests only
 BENCH_LIB = os.path.join(HERE, "libpolarquant_bench.so")
@@ -100,26 +105,28 @@ def build_probe(name: str, verbose: bool = True) -> str:
     return PROBE_LIB
 
 
-def build_latent(verbose: bool = True) -> str:
-    """libpolarquant_latent.so alone."""
+def build_layers(names=tuple(LAYER_UNITS), verbose: bool = True) -> None:
+    """The named libraries of LAYER_UNITS alone."""
     os.makedirs(OBJ, exist_ok=True)
-    with ThreadPoolExecutor(max_workers=len(LATENT_UNITS)) as ex:
-        objs = list(ex.map(lambda j: _compile(*j), LATENT_UNITS))
-    _link(objs, LATENT_LIB)
-    if verbose:
-        print("built", LATENT_LIB)
-    return LATENT_LIB
+    units = [u for n in names for u in LAYER_UNITS[n]]
+    with ThreadPoolExecutor(max_workers=min(8, max(len(units), 1))) as ex:
+        built = dict(zip(units, ex.map(lambda j: _compile(*j), units)))
+    for n in names:
+        _link([built[u] for u in LAYER_UNITS[n]], LAYER_LIBS[n])
+        if verbose:
+            print("built", LAYER_LIBS[n])
 
 
-LIBRARIES = {"hip": LIB, "latent": LATENT_LIB}
+LIBRARIES = dict(LAYER_LIBS, hip=LIB)
 
 
 def ensure(libraries, verbose: bool = True) -> None:
     """Build those of the named LIBRARIES that are not there, and nothing else."""
     if "hip" in libraries and not os.path.exists(LIB):
         build(verbose)
-    if "latent" in libraries and not os.path.exists(LATENT_LIB):
-        build_latent(verbose)
+    missing = [n for n in libraries if n in LAYER_LIBS and not os.path.exists(LAYER_LIBS[n])]
+    if missing:
+        build_layers(missing, verbose)
 
 
 def build(verbose: bool = True, phase_timers: bool = False) -> str:
@@ -134,7 +141,7 @@ def build(verbose: bool = True, phase_timers: bool = False) -> str:
         main = list(UNITS)
         hooks = [HOOKS_UNITS.get((src, tag), (src, defs, tag)) for src, defs, tag in UNITS]
         bench = [(s_, (), "") for s_ in BENCH_SOURCES]
-        jobs = main + [u for u in hooks if u not in main] + LATENT_UNITS + bench
+        jobs = main + [u for u in hooks if u not in main] + [u for us in LAYER_UNITS.values() for u in us] + bench
     # the units are listed longest compilation first
     with ThreadPoolExecutor(max_workers=min(8, len(jobs))) as ex:
         built = dict(zip(jobs, ex.map(lambda j: _compile(*j), jobs)))
@@ -142,10 +149,12 @@ def build(verbose: bool = True, phase_timers: bool = False) -> str:
     _link([built[u] for u in main], lib)
     if not phase_timers:
         _link([built[u] for u in hooks], HOOKS_LIB)
-        _link([built[u] for u in LATENT_UNITS], LATENT_LIB)
+        for name, units in LAYER_UNITS.items():
+            _link([built[u] for u in units], LAYER_LIBS[name])
         _link([built[u] for u in bench], BENCH_LIB)
         if verbose:
-            print("built", LATENT_LIB)
+            for path in LAYER_LIBS.values():
+                print("built", path)
             print("built", HOOKS_LIB)
             print("built", BENCH_LIB)
     if verbose:
@@ -156,7 +165,7 @@ def build(verbose: bool = True, phase_timers: bool = False) -> str:
 if __name__ == "__main__":
     if "--probe" in sys.argv[1:]:
         build_probe(sys.argv[sys.argv.index("--probe") + 1])
-    elif "--latent" in sys.argv[1:]:
-        build_latent()
+    elif "--layers" in sys.argv[1:]:
+        build_layers(sys.argv[sys.argv.index("--layers") + 1:] or tuple(LAYER_UNITS))
     else:
         build(phase_timers="--phase-timers" in sys.argv[1:])

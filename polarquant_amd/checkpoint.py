@@ -15,7 +15,7 @@ from __future__ import annotations
 import dataclasses
 import json
 import os
-from typing import Dict, Iterable, List, Optional
+from typing import Dict, Iterable, List, Optional, Tuple
 
 import torch
 
@@ -78,6 +78,15 @@ def _shard_files(path: str) -> List[str]:
     raise FileNotFoundError("polarquant_amd: no model.safetensors(.index.json) in %s (pickle checkpoints are not read)" % path)
 
 
+def _tensor_shapes(shard_files: Iterable[str]) -> Dict[str, Tuple[int, ...]]:
+    from safetensors import safe_open
+    out = {}
+    for fn in shard_files:
+        with safe_open(fn, framework="pt", device="cpu") as f:
+            out.update({name: tuple(f.get_slice(name).get_shape()) for name in f.keys()})
+    return out
+
+
 def _named_tensors(model: torch.nn.Module) -> Dict[str, torch.nn.Parameter]:
     """Checkpoint tensor name -> parameter: the module paths, unless the model maps its names itself."""
     own = getattr(model, "checkpoint_tensors", None)
@@ -125,6 +134,9 @@ def load_pretrained(path: str, dtype: torch.dtype = torch.bfloat16, device="cuda
         d = json.load(f)
     family = family_of(d)
     cfg = family.config(d, **options)
+    files = _shard_files(path)
+    if hasattr(cfg, "take_shapes"):                 # sizes that only the tensors tell
+        cfg.take_shapes(_tensor_shapes(files))
     prev = torch.get_default_dtype()
     torch.set_default_dtype(dtype)
     try:
@@ -132,7 +144,7 @@ def load_pretrained(path: str, dtype: torch.dtype = torch.bfloat16, device="cuda
             model = (model_class or family.model_class())(cfg)
     finally:
         torch.set_default_dtype(prev)
-    load_state(model, _shard_files(path), dtype)
+    load_state(model, files, dtype)
     return model.eval()
 
 

@@ -11,44 +11,10 @@
 // O^T = V^T P^T, takes its right operand in, once the tokens are numbered accordingly (the order of the summed index is
 // free as long as both operands agree).  Scores, their softmax and all sums are float32; latents, queries and weights
 // enter the products in the model's 16-bit dtype.
-#include "pq_device.h"
+#include "pq_mfma.h"
 #include "pq_latent_internal.h"
 
 namespace pq {
-
-struct F32 {};
-typedef float floatx4_a __attribute__((ext_vector_type(4)));
-typedef float floatx16_a __attribute__((ext_vector_type(16)));
-typedef uint32_t u32x4_a __attribute__((ext_vector_type(4)));
-typedef uint32_t u32x2_a __attribute__((ext_vector_type(2)));
-typedef _Float16 half8_a __attribute__((ext_vector_type(8)));
-typedef __bf16 bf16x8_a __attribute__((ext_vector_type(8)));
-typedef short short4_a __attribute__((ext_vector_type(4)));
-typedef __attribute__((address_space(3))) short4_a lds_short4;
-typedef __attribute__((address_space(3))) u32x4_a lds_u32x4;
-
-template <typename T> __device__ __forceinline__ floatx4_a mma16(u32x4_a a, u32x4_a b, floatx4_a c);
-template <> __device__ __forceinline__ floatx4_a mma16<F16>(u32x4_a a, u32x4_a b, floatx4_a c) {
-    return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(half8_a, a), __builtin_bit_cast(half8_a, b), c, 0, 0, 0);
-}
-template <> __device__ __forceinline__ floatx4_a mma16<BF16>(u32x4_a a, u32x4_a b, floatx4_a c) {
-    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_a, a), __builtin_bit_cast(bf16x8_a, b), c, 0, 0, 0);
-}
-template <typename T> __device__ __forceinline__ floatx16_a mma32(u32x4_a a, u32x4_a b, floatx16_a c);
-template <> __device__ __forceinline__ floatx16_a mma32<F16>(u32x4_a a, u32x4_a b, floatx16_a c) {
-    return __builtin_amdgcn_mfma_f32_32x32x16_f16(__builtin_bit_cast(half8_a, a), __builtin_bit_cast(half8_a, b), c, 0, 0, 0);
-}
-template <> __device__ __forceinline__ floatx16_a mma32<BF16>(u32x4_a a, u32x4_a b, floatx16_a c) {
-    return __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_a, a), __builtin_bit_cast(bf16x8_a, b), c, 0, 0, 0);
-}
-
-constexpr float kLog2e = 1.4426950408889634f;
-constexpr float kNone = -1.0e30f;         // running maximum before any key
-__device__ __forceinline__ float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
-
-template <typename T> __device__ __forceinline__ uint32_t pack2(float a, float b) {
-    return static_cast<uint32_t>(f2lo<T>(a)) | (static_cast<uint32_t>(f2lo<T>(b)) << 16);
-}
 
 // ---- decode --------------------------------------------------------------------------------------------------------
 // grid (slices, row tiles, sequences); a row is (query token, head), a workgroup owns 16 * RT of them and walks its slice

@@ -20,10 +20,10 @@
 //
 // EPI 0 is the kernel as described (bias, or the gated form); EPI 1 + e is the same stream for one of `heads` independent
 // products per launch (blockIdx.y == head, operands `x_head` / N * K / `y_head` elements apart) with epilogue e of
-// pq_latent_internal.h: plain, square of relu, times sigmoid(gate), or unrounded float32 output.
+// pq_steps_internal.h: plain, square of relu, times sigmoid(gate), or unrounded float32 output.
 #pragma once
 #include "pq_device.h"
-#include "pq_latent_internal.h"
+#include "pq_steps_internal.h"
 
 namespace pq {
 

@@ -1,63 +1,19 @@
-// The steps around latent attention: norms, input convolution, projections of small batches.
+// The steps between a layer's mixers and matrix products, whatever the mixers are.
 //
 //   norm_conv_kernel    residual add of a normed sublayer output, grouped RMS norm of the sum, causal convolution over
 //                       time with its per-sequence state: everything between two sublayers in one launch
-//   latent_norm_kernel  RMS norms of the query latent and of the key/value latent, the latter written to its cache row
+//   stream_add_kernel   residual stream + sublayer output + another stream + one vector
+//   embed_rows_kernel   scaled embedding rows as the float32 stream
 //   relu_sq_kernel      square of relu
+//   gelu_mul_kernel     gelu (tanh form) of one product times another
+//   softcap_kernel      scale and soft cap of logits
 //   head_linear_kernel  per-head (or plain) matrix product for sizes and dtypes the matrix-core kernels do not take
 //
 // All of this is fp32 arithmetic on whatever the operands' dtype is; results are rounded to it once.
-#include "pq_device.h"
-#include "pq_latent_internal.h"
+#include "pq_elem.h"
+#include "pq_steps_internal.h"
 
 namespace pq {
-
-struct F32 {};
-
-template <typename T> struct Elem { using type = uint16_t; };
-template <> struct Elem<F32> { using type = float; };
-template <typename T> using elem_t = typename Elem<T>::type;
-
-template <typename T> __device__ __forceinline__ float ld1(const elem_t<T>* p) {
-    if constexpr (__is_same(T, F32)) return *p; else return lo2f<T>(*p);
-}
-template <typename T> __device__ __forceinline__ elem_t<T> cv1(float f) {
-    if constexpr (__is_same(T, F32)) return f; else return f2lo<T>(f);
-}
-// V consecutive elements (V 1 or 4; for 4 the address is a multiple of 4 elements)
-template <typename T, int V> __device__ __forceinline__ void ldv(const void* base, size_t i, float (&o)[V]) {
-    const elem_t<T>* p = static_cast<const elem_t<T>*>(base) + i;
-    if constexpr (V == 1) {
-        o[0] = ld1<T>(p);
-    } else if constexpr (__is_same(T, F32)) {
-        const float4 v = *reinterpret_cast<const float4*>(p);
-        o[0] = v.x; o[1] = v.y; o[2] = v.z; o[3] = v.w;
-    } else {
-        const uint2 v = *reinterpret_cast<const uint2*>(p);
-        o[0] = lo2f<T>(static_cast<uint16_t>(v.x & 0xffffu)); o[1] = lo2f<T>(static_cast<uint16_t>(v.x >> 16));
-        o[2] = lo2f<T>(static_cast<uint16_t>(v.y & 0xffffu)); o[3] = lo2f<T>(static_cast<uint16_t>(v.y >> 16));
-    }
-}
-template <typename T, int V> __device__ __forceinline__ void stv(void* base, size_t i, const float (&o)[V]) {
-    elem_t<T>* p = static_cast<elem_t<T>*>(base) + i;
-    if constexpr (V == 1) {
-        *p = cv1<T>(o[0]);
-    } else if constexpr (__is_same(T, F32)) {
-        *reinterpret_cast<float4*>(p) = make_float4(o[0], o[1], o[2], o[3]);
-    } else {
-        *reinterpret_cast<uint2*>(p) = make_uint2(static_cast<uint32_t>(f2lo<T>(o[0])) | (static_cast<uint32_t>(f2lo<T>(o[1])) << 16),
-                                                  static_cast<uint32_t>(f2lo<T>(o[2])) | (static_cast<uint32_t>(f2lo<T>(o[3])) << 16));
-    }
-}
-
-// sum over the wavefront, in every lane: rotations inside rows of 16 lanes, then the four rows' sums through scalars
-__device__ __forceinline__ float wave_sum(float v) {
-    v += __uint_as_float(row_rotate<8>(__float_as_uint(v)));
-    v += __uint_as_float(row_rotate<4>(__float_as_uint(v)));
-    v += __uint_as_float(row_rotate<2>(__float_as_uint(v)));
-    v += __uint_as_float(row_rotate<1>(__float_as_uint(v)));
-    return (readlane_f(v, 0) + readlane_f(v, 16)) + (readlane_f(v, 32) + readlane_f(v, 48));
-}
 
 // ---- residual add + grouped norms + causal convolution ----------------------------------------------------------------
 // A workgroup walks a strip of consecutive tokens of one sequence; a thread owns the same NC pieces of V channels for all
@@ -174,7 +130,7 @@ __global__ __launch_bounds__(512) void norm_conv_kernel(NormConvArgs a) {
 #pragma unroll
     for (int k = 0; k < NC; k++) {
         ldv<T, V>(a.w_pre, ch[k], wpre[k]);
-        ldv<T, V>(a.y ? a.w_post : a.w_pre, ch[k], wpost[k]);
+        ldv<T, V>(a.w_post ? a.w_post : a.w_pre, ch[k], wpost[k]);
     }
     // (loads of what a shorter filter or a later strip does not have go to an address that exists and are dropped: with a
     // branch around each, every one would be waited for before the next)
@@ -223,12 +179,19 @@ __global__ __launch_bounds__(512) void norm_conv_kernel(NormConvArgs a) {
     for (int t = begin; t < t1; t++) {
         const size_t row = (static_cast<size_t>(b) * L + t) * W;
         if (a.y) {
-            float r[NC];
-            group_scale(yc, r);
+            if (a.w_post) {
+                float r[NC];
+                group_scale(yc, r);
 #pragma unroll
-            for (int k = 0; k < NC; k++)
+                for (int k = 0; k < NC; k++)
 #pragma unroll
-                for (int i = 0; i < V; i++) xc[k][i] = __builtin_fmaf(wpost[k][i], yc[k][i] * r[k], xc[k][i]);
+                    for (int i = 0; i < V; i++) xc[k][i] = __builtin_fmaf(wpost[k][i], yc[k][i] * r[k], xc[k][i]);
+            } else {
+#pragma unroll
+                for (int k = 0; k < NC; k++)
+#pragma unroll
+                    for (int i = 0; i < V; i++) xc[k][i] += yc[k][i];
+            }
             if (t >= t0)
 #pragma unroll
                 for (int k = 0; k < NC; k++)
@@ -320,66 +283,6 @@ int launch_norm_conv(const NormConvArgs& args, int dtype, hipStream_t st) {
     return static_cast<int>(hipGetLastError());
 }
 
-// ---- norms of the two latents ---------------------------------------------------------------------------------------
-// A wavefront per token when there are many (WIDE false), a workgroup per token otherwise.
-template <typename T, int V, bool WIDE>
-__global__ __launch_bounds__(256) void latent_norm_kernel(LatentNormArgs a) {
-    __shared__ float part[2][4];
-    const int wv = threadIdx.x >> 6, n_tok = a.B * a.L;
-    const int first = (WIDE ? static_cast<int>(threadIdx.x) : static_cast<int>(threadIdx.x & 63)) * V, step = (WIDE ? 256 : 64) * V;
-    int tok = WIDE ? static_cast<int>(blockIdx.x) : static_cast<int>(blockIdx.x) * 4 + wv;
-    if (!WIDE && tok >= n_tok) return;
-    const int b = tok / a.L, t = tok - b * a.L;
-    const int Q = a.q_rank, R = a.w_kv ? a.kv_rank : 0;
-    const elem_t<T>* p = static_cast<const elem_t<T>*>(a.p) + static_cast<size_t>(tok) * a.row_stride;
-    float sq = 0.0f, sc = 0.0f, v[V];
-    for (int i = first; i < Q + R; i += step) {
-        ldv<T, V>(p, i, v);
-        float s = 0.0f;
-#pragma unroll
-        for (int j = 0; j < V; j++) s = __builtin_fmaf(v[j], v[j], s);
-        sq += i < Q ? s : 0.0f;
-        sc += i < Q ? 0.0f : s;
-    }
-    sq = wave_sum(sq);
-    sc = wave_sum(sc);
-    if (WIDE) {
-        if ((threadIdx.x & 63) == 0) { part[0][wv] = sq; part[1][wv] = sc; }
-        __syncthreads();
-        sq = part[0][0] + part[0][1] + part[0][2] + part[0][3];
-        sc = part[1][0] + part[1][1] + part[1][2] + part[1][3];
-    }
-    const float rq = rsqrtf(sq / static_cast<float>(Q) + a.eps), rc = R ? rsqrtf(sc / static_cast<float>(R) + a.eps) : 0.0f;
-    int64_t pos = (a.pos_dev ? *a.pos_dev : a.pos) + t;
-    pos = pos < 0 ? 0 : (pos >= a.capacity ? a.capacity - 1 : pos);          // (never past the cache)
-    elem_t<T>* qo = static_cast<elem_t<T>*>(a.q_out) + static_cast<size_t>(tok) * Q;
-    elem_t<T>* co = static_cast<elem_t<T>*>(a.cache) + (static_cast<size_t>(b) * a.capacity + pos) * R;
-    for (int i = first; i < Q + R; i += step) {
-        const bool is_q = i < Q;
-        float w[V];
-        ldv<T, V>(p, i, v);
-        ldv<T, V>(is_q ? a.w_q : a.w_kv, is_q ? i : i - Q, w);
-        const float r = is_q ? rq : rc;
-#pragma unroll
-        for (int j = 0; j < V; j++) v[j] = w[j] * (v[j] * r);
-        stv<T, V>(is_q ? qo : co, is_q ? i : i - Q, v);
-    }
-}
-
-int launch_latent_norm(const LatentNormArgs& a, int dtype, hipStream_t st) {
-    const bool v4 = a.q_rank % 4 == 0 && (!a.w_kv || a.kv_rank % 4 == 0) && a.row_stride % 4 == 0;
-    const int n_tok = a.B * a.L;
-    const bool wide = n_tok < 1024;
-    dim3 grid(static_cast<unsigned>(wide ? n_tok : (n_tok + 3) / 4)), block(256);
-#define PQ_LN1(T, V) do { if (wide) hipLaunchKernelGGL((latent_norm_kernel<T, V, true>), grid, block, 0, st, a); \
-                          else hipLaunchKernelGGL((latent_norm_kernel<T, V, false>), grid, block, 0, st, a); } while (0)
-#define PQ_LN(T) do { if (v4) PQ_LN1(T, 4); else PQ_LN1(T, 1); } while (0)
-    if (dtype == 0) PQ_LN(F16); else if (dtype == 1) PQ_LN(BF16); else PQ_LN(F32);
-#undef PQ_LN
-#undef PQ_LN1
-    return static_cast<int>(hipGetLastError());
-}
-
 // ---- square of relu ----------------------------------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void relu_sq_kernel(const void* __restrict__ x, void* __restrict__ y, size_t n) {
@@ -407,6 +310,97 @@ int launch_relu_sq(const void* x, void* y, size_t n, int dtype, hipStream_t st) 
     if (dtype == 0) hipLaunchKernelGGL(relu_sq_kernel<F16>, grid, block, 0, st, x, y, n);
     else if (dtype == 1) hipLaunchKernelGGL(relu_sq_kernel<BF16>, grid, block, 0, st, x, y, n);
     else hipLaunchKernelGGL(relu_sq_kernel<F32>, grid, block, 0, st, x, y, n);
+    return static_cast<int>(hipGetLastError());
+}
+
+// ---- gelu (tanh form) times --------------------------------------------------------------------------------------------
+// 0.5 z (1 + tanh u) = z / (1 + exp(-2 u)), u = sqrt(2 / pi) (z + 0.044715 z^3)
+__device__ __forceinline__ float gelu_tanh(float z) {
+    const float u2 = 1.5957691216057308f * (z + 0.044715f * z * z * z);
+    return z / (1.0f + expf(-u2));
+}
+
+// grid (column pieces, rows)
+template <typename T, int V>
+__global__ __launch_bounds__(256) void gelu_mul_kernel(GeluMulArgs a) {
+    const int c = (blockIdx.x * 256 + threadIdx.x) * V;
+    if (c >= a.cols) return;
+    for (int64_t row = blockIdx.y; row < a.rows; row += gridDim.y) {
+        float g[V], u[V];
+        ldv<T, V>(a.gate, row * a.in_stride + c, g);
+        ldv<T, V>(a.up, row * a.in_stride + c, u);
+#pragma unroll
+        for (int j = 0; j < V; j++) u[j] *= gelu_tanh(g[j]);
+        stv<T, V>(a.y, row * a.out_stride + c, u);
+    }
+}
+
+int launch_gelu_mul(const GeluMulArgs& a, int dtype, hipStream_t st) {
+    const size_t align = dtype == 2 ? 16 : 8;
+    auto ok = [&](const void* p) { return reinterpret_cast<uintptr_t>(p) % align == 0; };
+    const bool v4 = a.cols % 4 == 0 && a.in_stride % 4 == 0 && a.out_stride % 4 == 0 && ok(a.gate) && ok(a.up) && ok(a.y);
+    const int per = v4 ? 1024 : 256;
+    dim3 grid(static_cast<unsigned>((a.cols + per - 1) / per), static_cast<unsigned>(a.rows < 32768 ? a.rows : 32768)), block(256);
+#define PQ_GM(T) do { if (v4) hipLaunchKernelGGL((gelu_mul_kernel<T, 4>), grid, block, 0, st, a); \
+                      else hipLaunchKernelGGL((gelu_mul_kernel<T, 1>), grid, block, 0, st, a); } while (0)
+    if (dtype == 0) PQ_GM(F16); else if (dtype == 1) PQ_GM(BF16); else PQ_GM(F32);
+#undef PQ_GM
+    return static_cast<int>(hipGetLastError());
+}
+
+// ---- streams --------------------------------------------------------------------------------------------------------------
+// x_out = x (+ y) (+ e) (+ v), v one vector for every row.  grid (column pieces, rows)
+template <typename T>
+__global__ __launch_bounds__(256) void stream_add_kernel(StreamAddArgs a) {
+    const int c = blockIdx.x * 256 + threadIdx.x;
+    if (c >= a.width) return;
+    const float v = a.v ? ld1<T>(static_cast<const elem_t<T>*>(a.v) + c) : 0.0f;
+    for (int64_t row = blockIdx.y; row < a.rows; row += gridDim.y) {
+        const size_t i = static_cast<size_t>(row) * a.width + c;
+        float x = a.x[i];
+        if (a.y) x += ld1<T>(static_cast<const elem_t<T>*>(a.y) + i);
+        if (a.e) x += a.e[i];
+        a.x_out[i] = x + v;
+    }
+}
+
+int launch_stream_add(const StreamAddArgs& a, int dtype, hipStream_t st) {
+    dim3 grid(static_cast<unsigned>((a.width + 255) / 256), static_cast<unsigned>(a.rows < 32768 ? a.rows : 32768)), block(256);
+    if (dtype == 0) hipLaunchKernelGGL(stream_add_kernel<F16>, grid, block, 0, st, a);
+    else if (dtype == 1) hipLaunchKernelGGL(stream_add_kernel<BF16>, grid, block, 0, st, a);
+    else hipLaunchKernelGGL(stream_add_kernel<F32>, grid, block, 0, st, a);
+    return static_cast<int>(hipGetLastError());
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void embed_rows_kernel(const void* table, const int64_t* ids, float scale, float* out, int64_t rows, int width, int64_t vocab) {
+    const int c = blockIdx.x * 256 + threadIdx.x;
+    if (c >= width) return;
+    for (int64_t row = blockIdx.y; row < rows; row += gridDim.y) {
+        int64_t id = ids[row];
+        id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);          // (never past the table)
+        out[static_cast<size_t>(row) * width + c] = ld1<T>(static_cast<const elem_t<T>*>(table) + static_cast<size_t>(id) * width + c) * scale;
+    }
+}
+
+int launch_embed_rows(const void* table, const int64_t* ids, float scale, float* out, int64_t rows, int width, int64_t vocab, int dtype, hipStream_t st) {
+    dim3 grid(static_cast<unsigned>((width + 255) / 256), static_cast<unsigned>(rows < 32768 ? rows : 32768)), block(256);
+    if (dtype == 0) hipLaunchKernelGGL(embed_rows_kernel<F16>, grid, block, 0, st, table, ids, scale, out, rows, width, vocab);
+    else if (dtype == 1) hipLaunchKernelGGL(embed_rows_kernel<BF16>, grid, block, 0, st, table, ids, scale, out, rows, width, vocab);
+    else hipLaunchKernelGGL(embed_rows_kernel<F32>, grid, block, 0, st, table, ids, scale, out, rows, width, vocab);
+    return static_cast<int>(hipGetLastError());
+}
+
+// ---- logits ---------------------------------------------------------------------------------------------------------------
+__global__ __launch_bounds__(256) void softcap_kernel(float* x, size_t n, float scale, float cap) {
+    const size_t i = static_cast<size_t>(blockIdx.x) * 256 + threadIdx.x;
+    if (i >= n) return;
+    const float z = x[i] * scale;
+    x[i] = cap > 0.0f ? cap * tanhf(z / cap) : z;
+}
+
+int launch_softcap(float* x, size_t n, float scale, float cap, hipStream_t st) {
+    hipLaunchKernelGGL(softcap_kernel, dim3(static_cast<unsigned>((n + 255) / 256)), dim3(256), 0, st, x, n, scale, cap);
     return static_cast<int>(hipGetLastError());
 }
 

@@ -328,8 +328,8 @@ class PolarGraphDecoder(GraphDecoder):
         return tuple(ar.as_tuple() for ar in self.arenas)
 
 
-class LatentGraphDecoder(GraphDecoder):
-    """The same for latent-attention models (`modeling_latent`): the step is the model's own `run` for one token, with the
+class LayeredGraphDecoder(GraphDecoder):
+    """The same for models on the `modeling_layered` shell: the step is the model's own `run` for one token, with the
     position in device memory."""
 
     def __init__(self, model, max_len: int, use_graph: bool = True):
@@ -337,7 +337,6 @@ class LatentGraphDecoder(GraphDecoder):
 
     @torch.no_grad()
     def prefill(self, input_ids: torch.Tensor, attention_mask: Optional[torch.Tensor] = None) -> torch.Tensor:
-        from .latent_ops import decode_splits
         B, L = input_ids.shape
         assert L + 1 <= self.max_len
         out = self.model(input_ids=input_ids, attention_mask=attention_mask, num_logits_to_keep=1,
@@ -347,14 +346,14 @@ class LatentGraphDecoder(GraphDecoder):
         dev = input_ids.device
         self.pos = torch.full((1,), L, dtype=torch.int32, device=dev)
         self.ids = torch.zeros((B, 1), dtype=torch.long, device=dev)
-        self.n_splits = [decode_splits(B, 1, layer.mix.heads, self.max_len, dev) for layer in self.model.model.layers]
+        self.plan = self.model.model.step_plan(B, self.max_len, dev)
         return out.logits
 
     def _step_state(self):
-        return [self.pos] + [s.rows for a in self.arenas for s in a.conv]
+        return [self.pos] + [s for a in self.arenas for s in a.step_state()]
 
     def _step_body(self):
-        h = self.model.model.run(self.ids, self.arenas, 0, self.pos, self.n_splits)
+        h = self.model.model.run(self.ids, self.arenas, 0, self.pos, self.plan)
         logits = self.model.logits(h)
         self.pos.add_(1)
         return logits

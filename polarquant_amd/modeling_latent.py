@@ -1,4 +1,4 @@
-"""Decoder layers with latent attention: the mechanisms, their per-layer cache, and the model shell that runs them.
+"""Decoder layers with latent attention: the mechanisms, their per-layer cache, and the model that runs them.
 
 Mechanisms, each a module with its constants as arguments: `LatentAttention` (queries and a shared key/value latent
 through low-rank projections, no positions, a per-head sink, an output gate, optionally the latent of an earlier layer),
@@ -6,8 +6,7 @@ through low-rank projections, no positions, a per-head sink, an output gate, opt
 (norm before and after each sublayer).  The residual stream is float32 whatever the model's dtype.
 
 The cache tuple of a layer is `(latents | None, mixer-convolution state, feed-forward-convolution state | None, kv_seq_len)`,
-a `PolarCache` whose arena owns the tensors; the model's forward takes prompts, portions of prompts of any length, and
-single tokens alike.
+a `PolarCache` whose arena owns the tensors.
 """
 from __future__ import annotations
 
@@ -17,7 +16,8 @@ import torch
 import torch.nn as nn
 
 from . import latent_ops as ops
-from .modeling_common import PolarCache, PolarForCausalLM, CausalLMOutputWithPast
+from .modeling_common import PolarCache
+from .modeling_layered import LayeredForCausalLM, LayeredModel
 
 KEY_TILE = 64              # capacities are whole tiles of the prompt kernel's keys
 ABSORBED_TOKENS = 16       # up to this many new tokens per sequence, queries go to the latent space instead of keys and values to the heads'
@@ -56,6 +56,17 @@ class LatentArena:
         self.kv_len, self.start = 0, None
         for s in self.conv:
             s.reset()
+
+    def load(self, parts, n: int) -> None:
+        lat, *rows = parts
+        self.kv_len = n
+        if lat is not None:
+            self._c[:, :n] = lat
+        for state, r in zip(self.conv, rows):
+            state.rows.copy_(r)
+
+    def step_state(self) -> List[torch.Tensor]:
+        return [s.rows for s in self.conv]
 
     def as_tuple(self) -> PolarCache:
         lat = self._c[:, :self.kv_len] if self.source is None else None
@@ -173,22 +184,14 @@ class SandwichLayer(nn.Module):
             yield self.norm2, self.canon2, self.mlp, self.norm2b
 
 
-# ----------------------------------------------------------------------------- model shell
-class LatentModel(nn.Module):
-    """Embedding, `build_layers(config)`, final norm; `capture`, if a list, receives the residual stream after every layer."""
+# ----------------------------------------------------------------------------- model
+class LatentModel(LayeredModel):
+    """Layers with latent attention between an embedding and a final norm."""
 
     def __init__(self, config):
-        super().__init__()
-        self.config = config
-        self.embed_tokens = nn.Embedding(config.vocab_size, config.hidden_size)
-        self.layers = nn.ModuleList(self.build_layers(config))
+        super().__init__(config)
         self.norm = GroupRMSNorm(config.hidden_size, config.norm_groups, config.norm_eps)
-        self.capture: Optional[List[torch.Tensor]] = None
 
-    def build_layers(self, config):
-        raise NotImplementedError
-
-    # -- cache plumbing
     def new_arenas(self, B: int, capacity: int) -> List[LatentArena]:
         cfg, w = self.config, self.embed_tokens.weight
         arenas: List[LatentArena] = []
@@ -198,39 +201,12 @@ class LatentModel(nn.Module):
                                       None if a.kv_from is None else arenas[a.kv_from], layer.mlp is not None))
         return arenas
 
-    def _arenas_of(self, past_key_values, B: int) -> List[LatentArena]:
-        arenas = [getattr(t, "arena", None) for t in past_key_values]
-        if all(a is not None for a in arenas):
-            if any(a.kv_len != t[-1] for a, t in zip(arenas, past_key_values)):
-                raise ValueError("polarquant_amd: a cache of %d tokens was handed in whose state has moved on to %d (the convolutions' "
-                                 "states exist for the newest token only)" % (past_key_values[0][-1], arenas[0].kv_len))
-            return arenas
-        n = past_key_values[0][-1]                # plain tuples: copy them into fresh arenas
-        arenas = self.new_arenas(B, (self.config.cache_capacity or n + 1024))
-        for a, (lat, s1, s2, _) in zip(arenas, past_key_values):
-            a.kv_len = n
-            if lat is not None:
-                a.c[:, :n] = lat
-            for state, rows in zip(a.conv, (s1, s2)):
-                state.rows.copy_(rows)
-        return arenas
-
-    @staticmethod
-    def _left_padding(mask: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
-        """int32 [B] count of leading zeros of the mask [B, L], None if there are none."""
-        if mask is None:
-            return None
-        m = mask != 0
-        if bool(m.all()):
-            return None
-        if bool((m[:, 1:] < m[:, :-1]).any()):
-            raise ValueError("polarquant_amd: the attention mask may only mark left padding (zeros in front of ones)")
-        return (~m).sum(1).to(torch.int32)
+    def step_plan(self, B: int, max_len: int, device):
+        return [ops.decode_splits(B, 1, layer.mix.heads, max_len, device) for layer in self.layers]
 
     def run(self, input_ids: torch.Tensor, arenas: List[LatentArena], pos: int, pos_dev: Optional[torch.Tensor] = None,
-            n_splits: Optional[List[int]] = None) -> torch.Tensor:
-        """The layers over tokens [B, L] at positions pos .. (or *pos_dev ..): appends to the arenas' tensors and returns the
-        normed hidden states; the arenas' host counts are the caller's to advance."""
+            plan: Optional[List[int]] = None) -> torch.Tensor:
+        """plan: each layer's number of slices."""
         x = self.embed_tokens(input_ids).float()
         y = w_post = None
         start = arenas[0].start
@@ -241,7 +217,7 @@ class LatentModel(nn.Module):
                 if first_of_layer and i and self.capture is not None:
                     self.capture.append(x.clone())
                 if first_of_layer:
-                    y = sublayer(h, arena, pos, pos_dev, None if n_splits is None else n_splits[i])
+                    y = sublayer(h, arena, pos, pos_dev, None if plan is None else plan[i])
                 else:
                     y = sublayer(h)
                 w_post = post.weight
@@ -250,57 +226,9 @@ class LatentModel(nn.Module):
             self.capture.append(x.clone())
         return h
 
-    @torch.no_grad()
-    def forward(self, input_ids=None, attention_mask=None, past_key_values=None):
-        """-> (normed hidden states [B, L, W], tuple of per-layer cache tuples).  Any number of new tokens, with or without
-        a cache.  attention_mask [B, tokens so far] may mark left padding; it is read with the first tokens of a sequence."""
-        B, L = input_ids.shape
-        if past_key_values is None:
-            arenas, n = self.new_arenas(B, self.config.cache_capacity or L + 1024), 0
-        else:
-            arenas, n = self._arenas_of(past_key_values, B), past_key_values[0][-1]
-        if n == 0:
-            start = self._left_padding(attention_mask)
-            for a in arenas:
-                a.start = start
-        for a in arenas:
-            a.reserve(n + L)
-        h = self.run(input_ids, arenas, n)
-        for a in arenas:
-            a.kv_len = n + L
-        return h, tuple(a.as_tuple() for a in arenas)
 
-
-class LatentForCausalLM(PolarForCausalLM):
-    """The framework's causal-LM shell over a `LatentModel`; logits are float32."""
-
+class LatentForCausalLM(LayeredForCausalLM):
     model_class = LatentModel
-
-    def forward(self, input_ids=None, attention_mask=None, past_key_values=None, num_logits_to_keep=0, return_dict=True,
-                logit_positions: Optional[torch.Tensor] = None):
-        """logit_positions: indices into the new tokens whose logits are wanted, instead of the last num_logits_to_keep."""
-        h, past = self.model(input_ids=input_ids, attention_mask=attention_mask, past_key_values=past_key_values)
-        h = h[:, -num_logits_to_keep:] if logit_positions is None else h.index_select(1, logit_positions)
-        return CausalLMOutputWithPast(logits=self.logits(h), past_key_values=past)
-
-    @torch.no_grad()
-    def logits(self, h: torch.Tensor) -> torch.Tensor:
-        return ops.linear_f32(h.contiguous(), self.lm_head.weight)
-
-    def new_cache(self, batch: int, capacity: int):
-        """An empty cache of `capacity` tokens per sequence, to hand in as past_key_values."""
-        return tuple(a.as_tuple() for a in self.model.new_arenas(batch, capacity))
-
-    @staticmethod
-    def reset_cache(past_key_values):
-        """The cache's memory as an empty cache."""
-        for t in past_key_values:
-            t.arena.reset()
-        return tuple(t.arena.as_tuple() for t in past_key_values)
-
-    def graph_decoder(self, max_len: int):
-        from .graph_decode import LatentGraphDecoder
-        return LatentGraphDecoder(self, max_len)
 
     def kv_cache_bytes_per_token(self) -> int:
         """Latents only: the convolutions' states do not grow with the sequence."""

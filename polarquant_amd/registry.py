@@ -58,6 +58,17 @@ def _dekipel():
     return DekipelForCausalLM
 
 
+def _kapudra_config(d, **options):
+    from .modeling_kapudra import KapudraConfig
+    return KapudraConfig.from_dict(d, **options)
+
+
+def _kapudra():
+    from .modeling_kapudra import KapudraForCausalLM
+    return KapudraForCausalLM
+
+
 register(Family("llama", _polar_config, _llama, ("hip",), True), "llama", "mistral")      # (Mistral's layers are Llama's)
 register(Family("qwen2", _polar_config, _qwen2, ("hip",), True), "qwen2")
-register(Family("dekipel", _dekipel_config, _dekipel, ("latent",), False), "dekipel")
+register(Family("dekipel", _dekipel_config, _dekipel, ("steps", "latent"), False), "dekipel")
+register(Family("kapudra", _kapudra_config, _kapudra, ("steps", "recurrent"), False), "kapudra")

@@ -8,7 +8,7 @@ import torch
 
 from oracle import dekipel_oracle as do
 from polarquant_amd.checkpoint import load_generation_config, load_pretrained
-from polarquant_amd.graph_decode import LatentGraphDecoder
+from polarquant_amd.graph_decode import LayeredGraphDecoder
 from polarquant_amd.modeling_common import GenerationConfig, generate
 
 import dekipel_cases as dc
@@ -161,7 +161,7 @@ def test_graph_replays_equal_the_eager_step(gpu, tmp_path):
         mask[1, :7] = 0
         runs = []
         for use_graph in (True, False):
-            dec = LatentGraphDecoder(model, L + new + 1, use_graph=use_graph)
+            dec = LayeredGraphDecoder(model, L + new + 1, use_graph=use_graph)
             got = [dec.prefill(ids, mask)]
             for i in range(new):
                 got.append(dec.step(feed_ids[:, i:i + 1]).clone())

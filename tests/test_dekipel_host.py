@@ -56,7 +56,7 @@ def test_config_round_trip_and_registry():
         c = DekipelConfig.from_dict(cfg)
         assert c.to_dict() == cfg and DekipelConfig.from_dict(json.loads(json.dumps(c.to_dict()))) == c
     fam = family_of(dc.EVEN)
-    assert fam.model_class() is DekipelForCausalLM and not fam.polar_cache and fam.libraries == ("latent",)
+    assert fam.model_class() is DekipelForCausalLM and not fam.polar_cache and fam.libraries == ("steps", "latent")
     assert family_of({"model_type": "qwen2"}).name == "qwen2" and family_of({}).name == "llama"
     with pytest.raises(ValueError, match="not one of"):
         family_of({"architecture": "nobody"})
@@ -125,17 +125,27 @@ def test_left_padding_of_a_mask():
 # ---------------------------------------------------------------- C ABI argument checks
 @pytest.fixture(scope="module")
 def lib():
-    return _ffi.latent_lib()
+    class Both:                 # the steps' and the latent kernels' symbols
+        def __getattr__(self, name):
+            return getattr(_ffi.steps_lib() if name in _ffi.STEPS_SIGNATURES else _ffi.latent_lib(), name)
+    return Both()
 
 
 def test_header_and_signatures_name_the_same_symbols(lib):
     import os
     import re
     root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
-    with open(os.path.join(root, "include", "polarquant_latent.h")) as f:
-        text = re.sub(r"/\*.*?\*/", "", f.read(), flags=re.S)
-    names = set(re.findall(r"\b(pq_\w+)\s*\(", text))
-    assert names == set(_ffi.LATENT_SIGNATURES) and not names & set(_ffi.SIGNATURES)
+    seen = set(_ffi.SIGNATURES)
+    for header, table, load in (("steps", _ffi.STEPS_SIGNATURES, _ffi.steps_lib), ("latent", _ffi.LATENT_SIGNATURES, _ffi.latent_lib),
+                                ("recurrent", _ffi.RECURRENT_SIGNATURES, _ffi.recurrent_lib)):
+        with open(os.path.join(root, "include", "polarquant_%s.h" % header)) as f:
+            text = re.sub(r"/\*.*?\*/", "", f.read(), flags=re.S)
+        found = re.findall(r"\b(pq_\w+)\s*\(([^)]*)\)\s*;", text)
+        assert {n for n, _ in found} == set(table) and not seen & set(table)
+        for n, args in found:
+            assert len(args.split(",")) == len(table[n][1]), n
+        seen |= set(table)
+        load()
 
 
 A, B16 = 0x1000, 0x2000       # stand-in addresses; nothing is launched by the validators
@@ -150,7 +160,7 @@ def test_norm_conv_arguments(lib):
     assert call() == OK and call(dt=2) == OK and call(L=1, xo=A, so=A) == OK and call(cw=None, si=None, so=None, xo=A) == OK
     assert call(y=None, wp=None, xo=None) == OK and call(taps=1, si=None, so=None) == OK
     assert call(xo=A) == STRIDE and call(so=A) == STRIDE            # long calls are not in place
-    assert call(x=None) == NUL and call(wp=None) == NUL and call(si=None) == NUL
+    assert call(x=None) == NUL and call(xo=None) == NUL and call(wp=None) == OK and call(si=None) == NUL
     assert call(dt=3) == DTYPE and call(g=3) == SHAPE and call(W=0) == SHAPE and call(taps=17) == SHAPE and call(taps=0) == SHAPE
     assert call(W=16388, g=1) == SHAPE and call(W=4098, g=1) == SHAPE and call(W=16384, g=1) == OK
     assert call(x=A + 4) == ALIGN and call(B=0) == SHAPE and call(L=0) == SHAPE
