@@ -26,7 +26,8 @@
  * pq_memory_gates: log_i = cap tanh((i + b_i) / cap), log_f = log sigmoid(cap tanh((f + b_f) / cap)).
  * pq_memory_scan: m' = max(log_f + m, log_i); S <- exp(log_f + m - m') S + exp(log_i - m') k v^T,
  *   n alike with k alone; o = S^T q q_scale, den = max(|n . q| q_scale, exp(-m')) + 1e-6.
- *   state [B, H, vdim + 1, dim] (the last row is n), m [B, H].
+ *   state [B, H, vdim + 1, dim] (the last row is n), m [B, H, (vdim + 16) / 16]
+ *   (equal copies, one for every 16 state rows).
  * pq_head_norm_gate: out = out_scale * rmsnorm(o / den, per head) * w * sigmoid(gate);
  *   w [vdim] for all heads (w_head_stride 0) or [H * vdim] (w_head_stride vdim).
  */

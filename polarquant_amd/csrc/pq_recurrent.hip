@@ -171,7 +171,9 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs a) {
     float* sp = a.state + ((static_cast<size_t>(b) * H + h) * columns + (live ? col : 0)) * dim;
 #pragma unroll
     for (int i = 0; i < RPL; i++) S[i] = r0 + i < dim ? sp[r0 + i] : 0.0f;
-    float m = DELTA ? 0.0f : a.m[static_cast<size_t>(b) * H + h];
+    float* mp = DELTA ? nullptr : a.m + (static_cast<size_t>(b) * H + h) * gridDim.x + blockIdx.x;
+    float m = DELTA ? 0.0f : *mp;
+    if (!DELTA) __syncthreads();                     // (read by all before one writes it)
     const size_t row0 = static_cast<size_t>(b) * L;
     for (int t = 0; t < first; t++) {
         if (part == 0 && value) a.o[((row0 + t) * H + h) * a.vdim + col] = 0.0f;
@@ -252,7 +254,7 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs a) {
         for (int i = 0; i < RPL; i++)
             if (r0 + i < dim) sp[r0 + i] = S[i];
     }
-    if (!DELTA && col == a.vdim && part == 0) a.m[static_cast<size_t>(b) * H + h] = m;
+    if (!DELTA && threadIdx.x == 0) *mp = m;
 }
 
 template <bool DELTA>

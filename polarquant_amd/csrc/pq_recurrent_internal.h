@@ -92,7 +92,7 @@ struct ScanArgs {
     const float* beta;           // delta rule: [B * L, H]
     const float *log_i, *log_f;  // matrix memory: [B * L, H]
     float* state;                // [B, H, columns, dim]
-    float* m;                    // matrix memory: [B, H] running maximum
+    float* m;                    // matrix memory: [B, H, column blocks of 16] running maximum, one copy for each workgroup
     float* o;                    // [B * L, H, vdim]
     float* den;                  // matrix memory: [B * L, H]
     const int32_t* start;

@@ -124,8 +124,7 @@ class DeltaState:
 
 class MemoryState:
     def __init__(self, B: int, heads: int, dim: int, vdim: int, device):
-        self.S = torch.zeros(B, heads, vdim + 1, dim, dtype=torch.float32, device=device)       # the last row: the normalizer
-        self.m = torch.zeros(B, heads, dtype=torch.float32, device=device)
+        self.S, self.m = ops.memory_state(B, heads, dim, vdim, device)
 
     def tensors(self):
         return [self.S, self.m]

@@ -161,15 +161,22 @@ def memory_gates(i, f, b_i, b_f, cap: float):
     return li, lf
 
 
+def memory_state(B: int, heads: int, dim: int, vdim: int, device):
+    """A matrix memory's state at a sequence's start: matrices with the normalizer as their last row, running maxima (a copy
+    for every 16 rows, so that no workgroup of a launch reads what another writes)."""
+    return (torch.zeros(B, heads, vdim + 1, dim, dtype=torch.float32, device=device),
+            torch.zeros(B, heads, (vdim + 16) // 16, dtype=torch.float32, device=device))
+
+
 def memory_scan(q, k, v, log_i, log_f, state: torch.Tensor, m: torch.Tensor, q_scale: float, step: Step):
-    """Rows q, k [M, H * dim], v [M, H * vdim] of one projection; state [B, H, vdim + 1, dim] and m [B, H] float32, advanced in
+    """Rows q, k [M, H * dim], v [M, H * vdim] of one projection; state [B, H, vdim + 1, dim] and m as memory_state has them, advanced in
     place -> (o [M, H * vdim], den [M, H]) float32."""
     B, H, cols, dim = state.shape
     vdim, M, dt = cols - 1, step.B * step.L, _code(q)
     for t, n in ((q, H * dim), (k, H * dim), (v, H * vdim)):
         _rows(t, M, n, q.dtype)
         assert t.stride(0) == q.stride(0)
-    assert state.is_contiguous() and m.is_contiguous() and state.dtype == m.dtype == torch.float32 and m.shape == (B, H) and B == step.B
+    assert state.is_contiguous() and m.is_contiguous() and state.dtype == m.dtype == torch.float32 and m.shape == (B, H, (vdim + 16) // 16) and B == step.B
     assert log_i.shape == log_f.shape == (M, H) and log_i.is_contiguous() and log_f.is_contiguous()
     o = torch.empty(M, H * vdim, dtype=torch.float32, device=q.device)
     den = torch.empty(M, H, dtype=torch.float32, device=q.device)
