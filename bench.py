@@ -366,6 +366,8 @@ def main():
     ap.add_argument("--dekipel", action="store_true",
                     help="instead of the headline workload: prompt and decode throughput of the Dekipel decoder, and its kernels, beside the "
                          "Llama shell with the polar-key cache at equal size (one JSON line per figure)")
+    ap.add_argument("--kapudra", action="store_true",
+                    help="instead of the headline workload: the same for the Kapudra decoder (windowed attention, delta rule, matrix memories)")
     ap.add_argument("--copy-calib", action="store_true",
                     help="also run 3 plain 1 GiB device copies (torch clone): under `rocprofv3 --pmc FETCH_SIZE|WRITE_SIZE` "
                          "their counter values give the scale factor for the attention kernel's")
@@ -381,6 +383,10 @@ def main():
     if args.dekipel:
         from polarquant_amd.benchmarks import latent_bench
         latent_bench.main([])
+        return
+    if args.kapudra:
+        from polarquant_amd.benchmarks import recurrent_bench
+        recurrent_bench.main([])
         return
     from polarquant_amd import _ffi, workloads as wl
     if args.no_ramp:

@@ -28,6 +28,9 @@
  *   n alike with k alone; o = S^T q q_scale, den = max(|n . q| q_scale, exp(-m')) + 1e-6.
  *   state [B, H, vdim + 1, dim] (the last row is n), m [B, H, (vdim + 16) / 16]
  *   (equal copies, one for every 16 state rows).
+ *   Without a workspace both scans go token by token; with one, of pq_scan_workspace_bytes for
+ *   any number of tokens, 32 tokens at a time on the matrix cores, as many tokens ahead as it
+ *   holds (16-bit dtypes, no pos_dev).
  * pq_head_norm_gate: out = out_scale * rmsnorm(o / den, per head) * w * sigmoid(gate);
  *   w [vdim] for all heads (w_head_stride 0) or [H * vdim] (w_head_stride vdim).
  */
@@ -66,14 +69,16 @@ int pq_delta_prep(const void *q, const void *k, const void *v, const void *b, in
                   const void *dt_bias, const float *state_in, float *state_out, void *q_out, void *k_out, void *v_out,
                   float *q_inv, float *k_inv, float *log_g, float *beta, const int32_t *start, const int32_t *pos_dev, int pos,
                   int B, int L, int G, int H, int dim, int vdim, int taps, int dtype, void *stream);
+size_t pq_scan_workspace_bytes(int delta, int B, int H, int dim, int tokens, int dtype);
 int pq_delta_scan(const void *q, const void *k, const void *v, const float *q_inv, const float *k_inv, const float *log_g,
                   const float *beta, float *state, float *o, const int32_t *start, const int32_t *pos_dev, int pos, int B, int L,
-                  int G, int H, int dim, int vdim, int dtype, void *stream);
+                  int G, int H, int dim, int vdim, void *workspace, size_t workspace_bytes, int dtype, void *stream);
 int pq_memory_gates(const void *i, const void *f, int64_t row_stride, const void *b_i, const void *b_f, float *log_i,
                     float *log_f, int64_t rows, int H, float cap, int dtype, void *stream);
 int pq_memory_scan(const void *q, const void *k, const void *v, int64_t row_stride, const float *log_i, const float *log_f,
                    float *state, float *m, float *o, float *den, float q_scale, const int32_t *start, const int32_t *pos_dev,
-                   int pos, int B, int L, int H, int dim, int vdim, int dtype, void *stream);
+                   int pos, int B, int L, int H, int dim, int vdim, void *workspace, size_t workspace_bytes, int dtype,
+                   void *stream);
 int pq_head_norm_gate(const float *o, const float *den, const void *w, int w_head_stride, const void *gate,
                       int64_t gate_row_stride, void *out, int64_t out_row_stride, int64_t rows, int H, int vdim, float eps,
                       float out_scale, int dtype, void *stream);

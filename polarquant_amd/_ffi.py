@@ -136,9 +136,11 @@ RECURRENT_SIGNATURES = {
                        + [c_float, c_float, c_int, c_void_p, c_size_t, c_int, c_void_p]),
     "pq_validate_delta_prep": (c_int, [c_int] * 7 + [c_void_p, c_void_p, c_int64, c_int64, c_int]),
     "pq_delta_prep": (c_int, [c_void_p] * 4 + [c_int64, c_void_p, c_int64] + [c_void_p] * 16 + [c_int] * 9 + [c_void_p]),
-    "pq_delta_scan": (c_int, [c_void_p] * 11 + [c_int] * 8 + [c_void_p]),
+    "pq_scan_workspace_bytes": (c_size_t, [c_int] * 6),
+    "pq_delta_scan": (c_int, [c_void_p] * 11 + [c_int] * 7 + [c_void_p, c_size_t, c_int, c_void_p]),
     "pq_memory_gates": (c_int, [c_void_p, c_void_p, c_int64] + [c_void_p] * 4 + [c_int64, c_int, c_float, c_int, c_void_p]),
-    "pq_memory_scan": (c_int, [c_void_p] * 3 + [c_int64] + [c_void_p] * 6 + [c_float, c_void_p, c_void_p] + [c_int] * 7 + [c_void_p]),
+    "pq_memory_scan": (c_int, [c_void_p] * 3 + [c_int64] + [c_void_p] * 6 + [c_float, c_void_p, c_void_p] + [c_int] * 6
+                       + [c_void_p, c_size_t, c_int, c_void_p]),
     "pq_head_norm_gate": (c_int, [c_void_p] * 3 + [c_int, c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_int, c_float, c_float, c_int,
                                   c_void_p]),
 }

@@ -33,7 +33,8 @@ SOURCES = sorted({u[0] for u in UNITS})
 LAYER_UNITS = {
     "steps": [("pq_steps.hip", (), ""), ("pq_head_linear.hip", (), ""), ("pq_steps_capi.hip", (), "")],
     "latent": [("pq_latent_attn.hip", (), ""), ("pq_latent_norm.hip", (), ""), ("pq_latent_capi.hip", (), "")],
-    "recurrent": [("pq_window_attn.hip", (), ""), ("pq_recurrent.hip", (), ""), ("pq_recurrent_capi.hip", (), "")],
+    "recurrent": [("pq_window_attn.hip", (), ""), ("pq_recurrent_chunk.hip", (), ""), ("pq_recurrent.hip", (), ""),
+                  ("pq_recurrent_capi.hip", (), "")],
 }
 LAYER_LIBS = {name: os.path.join(HERE, "libpolarquant_%s.so" % name) for name in LAYER_UNITS}
 # measurement aids (a plain streaming read, the attention kernel's loads without its arithmetic): a library of

@@ -131,17 +131,34 @@ int pq_delta_prep(const void* q, const void* k, const void* v, const void* b, in
     return status(pq::launch_delta_prep(d, dtype, S(stream)));
 }
 
+size_t pq_scan_workspace_bytes(int delta, int B, int H, int dim, int tokens, int dtype) {
+    if (B < 1 || H < 1 || dim < 1 || dim > pq::kScanMaxDim || tokens < 1 || (dtype != PQ_F16 && dtype != PQ_BF16)) return 0;
+    const size_t chunks = (static_cast<size_t>(tokens) + pq::kRecurrentChunk - 1) / pq::kRecurrentChunk;
+    return chunks * B * H * pq::chunk_block_bytes(delta != 0, dim, dtype);
+}
+
+// a workspace asks for the chunked kernels
+static int check_chunks(bool delta, int B, int H, int dim, const void* workspace, size_t bytes, const int32_t* pos_dev, int dtype) {
+    if (pos_dev) return PQ_ERR_BAD_SHAPE;
+    if (dtype == PQ_F32) return PQ_ERR_BAD_DTYPE;
+    if (!aligned(workspace, 16)) return PQ_ERR_MISALIGNED;
+    return bytes < pq_scan_workspace_bytes(delta, B, H, dim, 1, dtype) ? PQ_ERR_WORKSPACE : PQ_OK;
+}
+
 int pq_delta_scan(const void* q, const void* k, const void* v, const float* q_inv, const float* k_inv, const float* log_g,
                   const float* beta, float* state, float* o, const int32_t* start, const int32_t* pos_dev, int pos, int B, int L, int G,
-                  int H, int dim, int vdim, int dtype, void* stream) {
+                  int H, int dim, int vdim, void* workspace, size_t workspace_bytes, int dtype, void* stream) {
     if (!q || !k || !v || !q_inv || !k_inv || !log_g || !beta || !state || !o) return PQ_ERR_NULL_POINTER;
     if (int rc = check_scan(B, L, G, H, dim, vdim, dtype)) return rc;
-    pq::ScanArgs a{};
+    if (workspace)
+        if (int rc = check_chunks(true, B, H, dim, workspace, workspace_bytes, pos_dev, dtype)) return rc;
+    pq::ChunkArgs a{};
+    a.workspace = static_cast<char*>(workspace);
     a.q = q; a.k = k; a.v = v;
     a.q_row = a.k_row = static_cast<int64_t>(G) * dim; a.v_row = static_cast<int64_t>(H) * vdim;
     a.q_inv = q_inv; a.k_inv = k_inv; a.log_g = log_g; a.beta = beta; a.state = state; a.o = o; a.start = start; a.pos_dev = pos_dev;
     a.pos = pos; a.B = B; a.L = L; a.G = G; a.H = H; a.dim = dim; a.vdim = vdim;
-    return status(pq::launch_delta_scan(a, dtype, S(stream)));
+    return status(workspace ? pq::launch_delta_chunks(a, workspace_bytes, dtype, S(stream)) : pq::launch_delta_scan(a, dtype, S(stream)));
 }
 
 int pq_memory_gates(const void* i, const void* f, int64_t row_stride, const void* b_i, const void* b_f, float* log_i, float* log_f,
@@ -156,16 +173,19 @@ int pq_memory_gates(const void* i, const void* f, int64_t row_stride, const void
 
 int pq_memory_scan(const void* q, const void* k, const void* v, int64_t row_stride, const float* log_i, const float* log_f, float* state,
                    float* m, float* o, float* den, float q_scale, const int32_t* start, const int32_t* pos_dev, int pos, int B, int L, int H,
-                   int dim, int vdim, int dtype, void* stream) {
+                   int dim, int vdim, void* workspace, size_t workspace_bytes, int dtype, void* stream) {
     if (!q || !k || !v || !log_i || !log_f || !state || !m || !o || !den) return PQ_ERR_NULL_POINTER;
     if (int rc = check_scan(B, L, H, H, dim, vdim, dtype)) return rc;
     if (row_stride < static_cast<int64_t>(H) * (dim > vdim ? dim : vdim)) return PQ_ERR_BAD_STRIDE;
-    pq::ScanArgs a{};
+    if (workspace)
+        if (int rc = check_chunks(false, B, H, dim, workspace, workspace_bytes, pos_dev, dtype)) return rc;
+    pq::ChunkArgs a{};
+    a.workspace = static_cast<char*>(workspace);
     a.q = q; a.k = k; a.v = v;
     a.q_row = a.k_row = a.v_row = row_stride;
     a.log_i = log_i; a.log_f = log_f; a.state = state; a.m = m; a.o = o; a.den = den; a.start = start; a.pos_dev = pos_dev;
     a.pos = pos; a.B = B; a.L = L; a.G = H; a.H = H; a.dim = dim; a.vdim = vdim; a.q_scale = q_scale;
-    return status(pq::launch_memory_scan(a, dtype, S(stream)));
+    return status(workspace ? pq::launch_memory_chunks(a, workspace_bytes, dtype, S(stream)) : pq::launch_memory_scan(a, dtype, S(stream)));
 }
 
 int pq_head_norm_gate(const float* o, const float* den, const void* w, int w_head_stride, const void* gate, int64_t gate_row_stride,

@@ -104,6 +104,16 @@ constexpr int kScanMaxDim = 256;
 int launch_delta_scan(const ScanArgs& a, int dtype, hipStream_t st);
 int launch_memory_scan(const ScanArgs& a, int dtype, hipStream_t st);
 
+// Both over many tokens, in chunks (pq_recurrent_chunk.hip): 16-bit dtypes, dim <= kScanMaxDim.
+constexpr int kRecurrentChunk = 32;
+struct ChunkArgs : ScanArgs {
+    char* workspace;             // [B, H, chunks] blocks of chunk_block_bytes
+    int t0, chunks;              // the segment: its first token in the call, how many chunks
+};
+size_t chunk_block_bytes(bool delta, int dim, int dtype);
+int launch_delta_chunks(const ChunkArgs& a, size_t workspace_bytes, int dtype, hipStream_t st);
+int launch_memory_chunks(const ChunkArgs& a, size_t workspace_bytes, int dtype, hipStream_t st);
+
 struct HeadNormGateArgs {
     const float* o;              // [rows, H, vdim]
     const float* den;            // [rows, H] divisors, or null

@@ -11,11 +11,13 @@ import torch
 from . import _ffi
 from .attention import _num_cus
 from .kernel4group import _stream_ptr
-from .layer_ops import ConvState, _code, _ptr
+from .layer_ops import _DTYPES, ConvState, _code, _ptr
 
 WINDOW_SMALL = 16          # new tokens per sequence up to which keys go to the ring before they are read
 MAX_DIM = 256              # of a recurrent head
 MAX_TAPS = 16
+CHUNKED_TOKENS = 64        # from this many tokens per sequence on, 16-bit recurrences run in chunks on the matrix cores
+WORKSPACE_BYTES = 160 << 20         # of a chunked recurrence, at most (what fits the last-level cache beside its other operands)
 
 
 class Step(NamedTuple):
@@ -99,6 +101,13 @@ def window_attention(q, ring: WindowRing, slopes: Optional[torch.Tensor], scale:
 
 
 # ----------------------------------------------------------------------------- gated delta rule
+def _scan_workspace(delta: bool, dtype: torch.dtype, step: Step, heads: int, dim: int, device) -> Optional[torch.Tensor]:
+    if dtype == torch.float32 or step.L < CHUNKED_TOKENS or step.pos_dev is not None:
+        return None
+    need = lambda tokens: _ffi.recurrent_lib().pq_scan_workspace_bytes(int(delta), step.B, heads, dim, tokens, _DTYPES[dtype])
+    return torch.empty(min(need(step.L), max(WORKSPACE_BYTES, need(1))), dtype=torch.uint8, device=device)
+
+
 class DeltaInputs(NamedTuple):
     q: torch.Tensor             # [M, G * dim] after convolution and silu
     k: torch.Tensor
@@ -142,8 +151,10 @@ def delta_scan(x: DeltaInputs, state: torch.Tensor, step: Step) -> torch.Tensor:
     assert state.is_contiguous() and state.dtype == torch.float32 and B == step.B and x.q.shape == (M, G * dim) and x.v.shape == (M, H * vdim)
     assert all(t.is_contiguous() for t in x) and x.log_g.shape == (M, H * dim) and x.beta.shape == (M, H)
     o = torch.empty(M, H * vdim, dtype=torch.float32, device=state.device)
+    ws = _scan_workspace(True, x.q.dtype, step, H, dim, state.device)
     _run(_ffi.recurrent_lib().pq_delta_scan, "pq_delta_scan", state.device, _ptr(x.q), _ptr(x.k), _ptr(x.v), _ptr(x.q_inv), _ptr(x.k_inv),
-         _ptr(x.log_g), _ptr(x.beta), _ptr(state), _ptr(o), _ptr(step.start), _ptr(step.pos_dev), step.pos, B, step.L, G, H, dim, vdim, dt)
+         _ptr(x.log_g), _ptr(x.beta), _ptr(state), _ptr(o), _ptr(step.start), _ptr(step.pos_dev), step.pos, B, step.L, G, H, dim, vdim,
+         _ptr(ws), 0 if ws is None else ws.numel(), dt)
     return o
 
 
@@ -180,8 +191,10 @@ def memory_scan(q, k, v, log_i, log_f, state: torch.Tensor, m: torch.Tensor, q_s
     assert log_i.shape == log_f.shape == (M, H) and log_i.is_contiguous() and log_f.is_contiguous()
     o = torch.empty(M, H * vdim, dtype=torch.float32, device=q.device)
     den = torch.empty(M, H, dtype=torch.float32, device=q.device)
+    ws = _scan_workspace(False, q.dtype, step, H, dim, q.device)
     _run(_ffi.recurrent_lib().pq_memory_scan, "pq_memory_scan", q.device, _ptr(q), _ptr(k), _ptr(v), q.stride(0), _ptr(log_i), _ptr(log_f),
-         _ptr(state), _ptr(m), _ptr(o), _ptr(den), float(q_scale), _ptr(step.start), _ptr(step.pos_dev), step.pos, B, step.L, H, dim, vdim, dt)
+         _ptr(state), _ptr(m), _ptr(o), _ptr(den), float(q_scale), _ptr(step.start), _ptr(step.pos_dev), step.pos, B, step.L, H, dim, vdim,
+         _ptr(ws), 0 if ws is None else ws.numel(), dt)
     return o, den
 
 
