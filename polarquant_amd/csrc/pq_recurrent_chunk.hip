@@ -13,8 +13,8 @@
 //
 //   delta_chunk_kernel, memory_chunk_kernel   what does not depend on the state, a workgroup per chunk and head, written
 //                                             in the order in which the matrix cores take their left operands
-//   delta_walk_kernel, memory_walk_kernel     the chunks in turn, a wavefront per head and 16 columns of the state, all in
-//                                             registers: no barrier, no LDS
+//   delta_walk_kernel, memory_walk_kernel     the chunks in turn, four wavefronts per head and 16 columns of the state,
+//                                             which stays in registers
 //
 // The products stand for float32 ones: each factor that is not a 16-bit number already is split into two bfloat16 numbers,
 // x = hi + lo, and hi hi + hi lo + lo hi is added up in float32 (what is left out is 2^-16 of a term).  State, decays,
@@ -257,12 +257,6 @@ __global__ __launch_bounds__(2 * DP) void delta_chunk_kernel(ChunkArgs a) {
 }
 
 // ---- delta rule, the chunks in turn --------------------------------------------------------------------------------------------
-template <typename T>
-__device__ __forceinline__ float value_at(const ChunkArgs& a, size_t row0, int t, int h, int col) {
-    const size_t row = row0 + (t < a.L ? t : a.L - 1);
-    return ld1<T>(static_cast<const elem_t<T>*>(a.v) + row * a.v_row + static_cast<size_t>(h) * a.vdim + col);
-}
-
 template <int NT> __device__ __forceinline__ void load_state(const float* sp, int dim, int g, floatx4_a (&S)[NT]) {
     static_for<NT>([&](auto J) {
         constexpr int j = decltype(J)::value;
@@ -284,131 +278,266 @@ template <int NT> __device__ __forceinline__ void store_state(float* sp, int dim
     });
 }
 
-// grid (column blocks of 16, heads, sequences), one wavefront.  Every operand is loaded again right after its use, a chunk ahead.
-template <typename T, int DP>
-__global__ __launch_bounds__(kWave, 1) void delta_walk_kernel(ChunkArgs a) {
-    using Blk = DeltaBlock<DP>;
-    constexpr int KS = DP / 32, NT = DP / 16;
-    const int lane = threadIdx.x, r16 = lane & 15, g = lane >> 4, h = blockIdx.y, b = blockIdx.z, H = a.H;
-    const int col = blockIdx.x * 16 + r16, cc = col < a.vdim ? col : a.vdim - 1;
-    const size_t row0 = static_cast<size_t>(b) * a.L;
-    const char* base = a.workspace + static_cast<size_t>(b * H + h) * a.chunks * Blk::size + lane * 16;
-    float* sp = a.state + ((static_cast<size_t>(b) * H + h) * a.vdim + cc) * a.dim;
-    floatx4_a S[NT];
-    load_state<NT>(sp, a.dim, g, S);
-
-    u32x4_a ki[2][2][KS], qi[2][2][KS], ko[2][NT], tm[2][2], pm[2][2];       // [part][row tile]..
-    floatx4_a dec[NT];
-    float v[2][4];
-    auto at = [&](const char* blk, int off) { return *reinterpret_cast<const u32x4_a*>(blk + off); };
-    auto load_ki = [&](const char* blk) {
-        static_for<2 * KS>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-            ki[0][i / KS][i % KS] = at(blk, Blk::k_in + i * 1024);
-            ki[1][i / KS][i % KS] = at(blk, Blk::k_in + Blk::kMat + i * 1024);
-        });
-    };
-    auto load_qi = [&](const char* blk) {
-        static_for<2 * KS>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-            qi[0][i / KS][i % KS] = at(blk, Blk::q_in + i * 1024);
-            qi[1][i / KS][i % KS] = at(blk, Blk::q_in + Blk::kMat + i * 1024);
-        });
-    };
-    auto load_ko = [&](const char* blk) {
-        static_for<NT>([&](auto J) {
-            constexpr int j = decltype(J)::value;
-            ko[0][j] = at(blk, Blk::k_out + j * 1024);
-            ko[1][j] = at(blk, Blk::k_out + Blk::kMat + j * 1024);
-            dec[j] = *reinterpret_cast<const floatx4_a*>(blk - lane * 16 + Blk::decay + (16 * j + 4 * g) * 4);
-        });
-    };
-    auto load_sq = [&](const char* blk) {
-        static_for<2>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-            tm[0][i] = at(blk, Blk::t + i * 1024);
-            tm[1][i] = at(blk, Blk::t + Blk::kSq + i * 1024);
-            pm[0][i] = at(blk, Blk::p + i * 1024);
-            pm[1][i] = at(blk, Blk::p + Blk::kSq + i * 1024);
-        });
-    };
-    auto load_v = [&](int t) {
+// A lane's four tokens of a row tile of a chunk, 16 rt + 4 g + i: their values as they are stored (converted when they are used,
+// so that nothing waits for them before).  Past the call's last token the last one is read.
+template <typename T> struct Rows {
+    const uint16_t* v;           // row 0 of the sequence's values, column 0 of the head
+    uint32_t stride, col;
+    int L, row;                  // row: the first of the four in the chunk
+    uint32_t off[4], raw[4];
+    __device__ __forceinline__ void offsets(int last) {
 #pragma unroll
-        for (int rt = 0; rt < 2; rt++)
-#pragma unroll
-            for (int i = 0; i < 4; i++) v[rt][i] = value_at<T>(a, row0, t + rt * 16 + 4 * g + i, h, cc);
-    };
-    load_v(a.t0);
-    load_ki(base);
-    load_qi(base);
-    load_sq(base);
-    load_ko(base);
-    for (int n = 0; n < a.chunks; n++) {
-        const int t = a.t0 + n * kChunk, next = n + 1 < a.chunks ? n + 1 : n;
-        const char* blk = base + static_cast<size_t>(next) * Blk::size;
-        u32x4_a sh[KS], sl[KS];
-        static_for<KS>([&](auto I) { constexpr int i = decltype(I)::value; split_tiles(S[2 * i], S[2 * i + 1], sh[i], sl[i]); });
-        floatx4_a R[2], R1[2], O[2], O1[2];
-#pragma unroll
-        for (int rt = 0; rt < 2; rt++) {
-            R[rt] = floatx4_a{v[rt][0], v[rt][1], v[rt][2], v[rt][3]};
-            R1[rt] = O[rt] = O1[rt] = floatx4_a{0, 0, 0, 0};
-        }
-        load_v(a.t0 + next * kChunk);
-        static_for<KS>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-#pragma unroll
-            for (int rt = 0; rt < 2; rt++) {
-                R[rt] = mm(ki[0][rt][i], sh[i], R[rt]);
-                R1[rt] = mm(ki[0][rt][i], sl[i], R1[rt]);
-                R1[rt] = mm(ki[1][rt][i], sh[i], R1[rt]);
-            }
-        });
-        load_ki(blk);
-        static_for<KS>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-#pragma unroll
-            for (int rt = 0; rt < 2; rt++) {
-                O[rt] = mm(qi[0][rt][i], sh[i], O[rt]);
-                O1[rt] = mm(qi[0][rt][i], sl[i], O1[rt]);
-                O1[rt] = mm(qi[1][rt][i], sh[i], O1[rt]);
-            }
-        });
-        load_qi(blk);
-        u32x4_a xh, xl;
-        split_tiles(R[0] + R1[0], R[1] + R1[1], xh, xl);
-        floatx4_a U[2], U1[2];
-#pragma unroll
-        for (int rt = 0; rt < 2; rt++) {
-            const floatx4_a zero = {0, 0, 0, 0};
-            U[rt] = mm(tm[0][rt], xh, zero);
-            U1[rt] = mm(tm[0][rt], xl, zero);
-            U1[rt] = mm(tm[1][rt], xh, U1[rt]);
-        }
-        static_for<NT>([&](auto J) { constexpr int j = decltype(J)::value; S[j] *= dec[j]; });
-        split_tiles(U[0] + U1[0], U[1] + U1[1], xh, xl);
-#pragma unroll
-        for (int rt = 0; rt < 2; rt++) {
-            O[rt] = mm(pm[0][rt], xh, O[rt]);
-            O1[rt] = mm(pm[0][rt], xl, O1[rt]);
-            O1[rt] = mm(pm[1][rt], xh, O1[rt]);
-        }
-        load_sq(blk);
-        static_for<NT>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[0][j], xh, S[j]); });
-        static_for<NT>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[0][j], xl, S[j]); });
-        static_for<NT>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[1][j], xh, S[j]); });
-        load_ko(blk);
-        if (col < a.vdim) {
-#pragma unroll
-            for (int rt = 0; rt < 2; rt++)
-#pragma unroll
-                for (int i = 0; i < 4; i++) {
-                    const int tt = t + rt * 16 + 4 * g + i;
-                    if (tt < a.L) a.o[((row0 + tt) * H + h) * a.vdim + col] = O[rt][i] + O1[rt][i];
-                }
-        }
+        for (int i = 0; i < 4; i++) off[i] = static_cast<uint32_t>(row + i < last ? row + i : last) * stride + col;
     }
-    if (col < a.vdim) store_state<NT>(sp, a.dim, g, S);
+    __device__ __forceinline__ void load(int t) {
+        const uint16_t* base = v + static_cast<size_t>(t) * stride;
+        if (L - 1 - t < kChunk - 1) offsets(L - 1 - t);              // uniform: the sequence's last chunk
+#pragma unroll
+        for (int i = 0; i < 4; i++) raw[i] = base[off[i]];
+    }
+    __device__ __forceinline__ floatx4_a get() const {
+        return floatx4_a{lo2f<T>(static_cast<uint16_t>(raw[0])), lo2f<T>(static_cast<uint16_t>(raw[1])),
+                         lo2f<T>(static_cast<uint16_t>(raw[2])), lo2f<T>(static_cast<uint16_t>(raw[3]))};
+    }
+};
+template <typename T> __device__ __forceinline__ Rows<T> rows_of(const ChunkArgs& a, size_t row0, int h, int col, int row) {
+    Rows<T> r{static_cast<const uint16_t*>(a.v) + row0 * a.v_row + static_cast<size_t>(h) * a.vdim, static_cast<uint32_t>(a.v_row),
+              static_cast<uint32_t>(col), a.L, row, {}, {}};
+    r.offsets(kChunk);
+    return r;
+}
+// out: the chunk's first row; left: rows from there to the call's end
+__device__ __forceinline__ void store_rows(float* out, uint32_t stride, uint32_t col, int row, int left, const floatx4_a& x) {
+    const uint32_t off = row * stride + col;
+    if (left >= kChunk) {                                            // uniform
+#pragma unroll
+        for (int i = 0; i < 4; i++) (out + i * static_cast<size_t>(stride))[off] = x[i];
+    } else {
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+            if (row + i < left) (out + i * static_cast<size_t>(stride))[off] = x[i];
+    }
+}
+
+// Four wavefronts share a walk, one on each SIMD.  The first two carry the state along, half of the channels each, and leave in
+// LDS what the other two multiply by Q' and P for the results, a row tile each.  Loads stay in flight across the barriers.
+__device__ __forceinline__ void walk_barrier() {
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+}
+// chunks whose operands are in flight ahead of the one worked on, each in registers of its own
+constexpr int walk_ahead(int dp) { return dp <= 128 ? 2 : 1; }
+template <int AHEAD, typename F> __device__ __forceinline__ void walk_chunks(int chunks, F&& step) {
+    for (int n = 0; n < chunks; n += AHEAD)
+        static_for<AHEAD>([&](auto P) {
+            if (n + P < chunks) step(P, n + P);
+        });
+}
+
+// The workgroups of a head fetch the lines of a chunk still further ahead into their L2 in turn, one load each: the operands
+// come from the last-level cache or memory.  The value is dropped, a chunk's time or more after the load.
+struct LineFetch {
+    const char* base;
+    int block_bytes, ahead, chunks;
+    uint32_t off, got;
+    __device__ __forceinline__ void go(int n) {
+        const int m = n + ahead < chunks ? n + ahead : chunks - 1;
+        got = *reinterpret_cast<const uint32_t*>(base + static_cast<size_t>(m) * block_bytes + off);
+    }
+    __device__ __forceinline__ void drop() const { asm volatile("" ::"v"(got)); }
+};
+__device__ __forceinline__ LineFetch line_fetch(const char* base, int block_bytes, const ChunkArgs& a, int lane) {
+    const uint32_t off = static_cast<uint32_t>(lane * static_cast<int>(gridDim.y) + static_cast<int>(blockIdx.y)) * 128u, last = block_bytes - 4;
+    return LineFetch{base, block_bytes, a.prefetch, a.chunks, off < last ? off : last, 0u};
+}
+
+// grid (heads, column blocks of 16, sequences): with a multiple of 8 heads all columns of a head run on one XCD and read its
+// operands from one L2.  Every operand is loaded again right after its use (the scheduling barriers keep the compiler from
+// moving those loads to where their results are needed).  Two barriers per chunk: the halves of K' S are added up between
+// them, while the read-out multiplies the state; U follows the second.
+template <typename T, int DP>
+__global__ __launch_bounds__(4 * kWave, 1) void delta_walk_kernel(ChunkArgs a) {
+    using Blk = DeltaBlock<DP>;
+    constexpr int KS = DP / 32, KH = KS / 2, NH = DP / 32, AHEAD = walk_ahead(DP);
+    __shared__ u32x4_a sh_s[2][KS][kWave], sh_u[2][kWave];           // high and low parts
+    __shared__ floatx4_a sh_r[2][2][kWave];                          // [half][row tile]
+    const int lane = threadIdx.x & 63, wv = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), r16 = lane & 15, g = lane >> 4;
+    const int h = blockIdx.x, b = blockIdx.z, H = a.H, col = blockIdx.y * 16 + r16, cc = col < a.vdim ? col : a.vdim - 1;
+    const size_t row0 = static_cast<size_t>(b) * a.L;
+    const char* base = a.workspace + static_cast<size_t>(b * H + h) * a.chunks * Blk::size;
+    const uint32_t lane16 = lane * 16, g16 = g * 16;
+    auto at = [&](const char* blk, int off) { return *reinterpret_cast<const u32x4_a*>(blk + off + lane16); };
+    if (wv < 2) {
+        const int c0 = wv * (DP / 2);                                // this wavefront's first channel
+        float* sp = a.state + ((static_cast<size_t>(b) * H + h) * a.vdim + cc) * a.dim + c0;
+        floatx4_a S[NH], dec[AHEAD][NH];
+        load_state<NH>(sp, a.dim - c0, g, S);
+        u32x4_a ki[AHEAD][2][2][KH], ko[AHEAD][2][NH], tm[AHEAD][2][2];      // [chunk][part][row tile]..
+        Rows<T> v[AHEAD];                                            // of row tile wv
+        auto load_ki = [&](auto P, const char* blk) {
+            constexpr int p = decltype(P)::value;
+            static_for<2 * KH>([&](auto I) {
+                constexpr int i = decltype(I)::value, rt = i / KH, k = i % KH;
+                const char* src = blk + Blk::k_in + wv * KH * 1024;
+                ki[p][0][rt][k] = at(src, (rt * KS + k) * 1024);
+                ki[p][1][rt][k] = at(src, Blk::kMat + (rt * KS + k) * 1024);
+            });
+        };
+        auto load_ko = [&](auto P, const char* blk) {
+            constexpr int p = decltype(P)::value;
+            static_for<NH>([&](auto J) {
+                constexpr int j = decltype(J)::value;
+                const char* src = blk + Blk::k_out + wv * NH * 1024;
+                ko[p][0][j] = at(src, j * 1024);
+                ko[p][1][j] = at(src, Blk::kMat + j * 1024);
+            });
+        };
+        auto load_t = [&](auto P, const char* blk) {
+            constexpr int p = decltype(P)::value;
+            static_for<2>([&](auto I) {
+                constexpr int i = decltype(I)::value;
+                tm[p][0][i] = at(blk, Blk::t + i * 1024);
+                tm[p][1][i] = at(blk, Blk::t + Blk::kSq + i * 1024);
+            });
+        };
+        auto load_dec = [&](auto P, const char* blk) {
+            constexpr int p = decltype(P)::value;
+            static_for<NH>([&](auto J) {
+                constexpr int j = decltype(J)::value;
+                dec[p][j] = *reinterpret_cast<const floatx4_a*>(blk + Blk::decay + wv * NH * 64 + j * 64 + g16);
+            });
+        };
+        static_for<AHEAD>([&](auto P) {
+            constexpr int p = decltype(P)::value;
+            const int n = p < a.chunks ? p : a.chunks - 1;
+            const char* blk = base + static_cast<size_t>(n) * Blk::size;
+            v[p] = rows_of<T>(a, row0, h, cc, wv * 16 + 4 * g);
+            v[p].load(a.t0 + n * kChunk);
+            load_ki(P, blk);
+            load_dec(P, blk);
+            load_t(P, blk);
+            load_ko(P, blk);
+        });
+        auto step = [&](auto P, int n) {
+            constexpr int p = decltype(P)::value;
+            const int next = n + AHEAD < a.chunks ? n + AHEAD : a.chunks - 1;
+            const char* blk = base + static_cast<size_t>(next) * Blk::size;
+            const floatx4_a zero = {0, 0, 0, 0}, V = v[p].get();
+            floatx4_a R[2] = {wv == 0 ? V : zero, wv == 0 ? zero : V}, R1[2] = {zero, zero};
+            __builtin_amdgcn_sched_barrier(0);
+            v[p].load(a.t0 + next * kChunk);
+            __builtin_amdgcn_sched_barrier(0);
+            static_for<KH>([&](auto I) {
+                constexpr int i = decltype(I)::value;
+                u32x4_a hi, lo;
+                split_tiles(S[2 * i], S[2 * i + 1], hi, lo);
+                sh_s[0][wv * KH + i][lane] = hi;
+                sh_s[1][wv * KH + i][lane] = lo;
+#pragma unroll
+                for (int rt = 0; rt < 2; rt++) {
+                    R[rt] = mm(ki[p][0][rt][i], hi, R[rt]);
+                    R1[rt] = mm(ki[p][0][rt][i], lo, R1[rt]);
+                    R1[rt] = mm(ki[p][1][rt][i], hi, R1[rt]);
+                }
+                S[2 * i] *= dec[p][2 * i];
+                S[2 * i + 1] *= dec[p][2 * i + 1];
+            });
+#pragma unroll
+            for (int rt = 0; rt < 2; rt++) {
+                R[rt] += R1[rt];
+                sh_r[wv][rt][lane] = R[rt];
+            }
+            __builtin_amdgcn_sched_barrier(0);
+            load_ki(P, blk);
+            load_dec(P, blk);
+            __builtin_amdgcn_sched_barrier(0);
+            walk_barrier();
+            u32x4_a xh, xl;
+            split_tiles(R[0] + sh_r[1 - wv][0][lane], R[1] + sh_r[1 - wv][1][lane], xh, xl);
+            floatx4_a U[2], U1[2];
+#pragma unroll
+            for (int rt = 0; rt < 2; rt++) {
+                U[rt] = mm(tm[p][0][rt], xh, zero);
+                U1[rt] = mm(tm[p][0][rt], xl, zero);
+                U1[rt] = mm(tm[p][1][rt], xh, U1[rt]);
+            }
+            __builtin_amdgcn_sched_barrier(0);
+            load_t(P, blk);
+            __builtin_amdgcn_sched_barrier(0);
+            split_tiles(U[0] + U1[0], U[1] + U1[1], xh, xl);
+            if (wv == 0) {
+                sh_u[0][lane] = xh;
+                sh_u[1][lane] = xl;
+            }
+            static_for<NH>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[p][0][j], xh, S[j]); });
+            static_for<NH>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[p][0][j], xl, S[j]); });
+            static_for<NH>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[p][1][j], xh, S[j]); });
+            __builtin_amdgcn_sched_barrier(0);
+            load_ko(P, blk);
+            __builtin_amdgcn_sched_barrier(0);
+            walk_barrier();
+        };
+        walk_chunks<AHEAD>(a.chunks, step);
+        if (col < a.vdim) store_state<NH>(sp, a.dim - c0, g, S);
+    } else {
+        const int rt = wv - 2, row = rt * 16 + 4 * g;
+        float* op = a.o + (row0 * H + h) * a.vdim;
+        const uint32_t o_stride = static_cast<uint32_t>(H) * a.vdim;
+        u32x4_a qi[AHEAD][2][KS], pm[AHEAD][2];
+        auto load_q = [&](auto P, const char* blk) {
+            constexpr int p = decltype(P)::value;
+            static_for<KS>([&](auto I) {
+                constexpr int i = decltype(I)::value;
+                const char* src = blk + Blk::q_in + rt * KS * 1024;
+                qi[p][0][i] = at(src, i * 1024);
+                qi[p][1][i] = at(src, Blk::kMat + i * 1024);
+            });
+        };
+        auto load_p = [&](auto P, const char* blk) {
+            constexpr int p = decltype(P)::value;
+            pm[p][0] = at(blk + rt * 1024, Blk::p);
+            pm[p][1] = at(blk + rt * 1024, Blk::p + Blk::kSq);
+        };
+        static_for<AHEAD>([&](auto P) {
+            const char* blk = base + static_cast<size_t>(P < a.chunks ? static_cast<int>(P) : a.chunks - 1) * Blk::size;
+            load_q(P, blk);
+            load_p(P, blk);
+        });
+        LineFetch lines = line_fetch(base, Blk::size, a, lane);
+        lines.go(0);
+        auto step = [&](auto P, int n) {
+            constexpr int p = decltype(P)::value;
+            const int t = a.t0 + n * kChunk, next = n + AHEAD < a.chunks ? n + AHEAD : a.chunks - 1;
+            const char* blk = base + static_cast<size_t>(next) * Blk::size;
+            floatx4_a O = {0, 0, 0, 0}, O1 = {0, 0, 0, 0};
+            walk_barrier();
+            static_for<KS>([&](auto I) {
+                constexpr int i = decltype(I)::value;
+                const u32x4_a hi = sh_s[0][i][lane], lo = sh_s[1][i][lane];
+                O = mm(qi[p][0][i], hi, O);
+                O1 = mm(qi[p][0][i], lo, O1);
+                O1 = mm(qi[p][1][i], hi, O1);
+            });
+            __builtin_amdgcn_sched_barrier(0);
+            load_q(P, blk);
+            __builtin_amdgcn_sched_barrier(0);
+            walk_barrier();
+            const u32x4_a xh = sh_u[0][lane], xl = sh_u[1][lane];
+            O = mm(pm[p][0], xh, O);
+            O1 = mm(pm[p][0], xl, O1);
+            O1 = mm(pm[p][1], xh, O1);
+            __builtin_amdgcn_sched_barrier(0);
+            load_p(P, blk);
+            if (rt == 0) {
+                lines.drop();
+                lines.go(n + 1);
+            }
+            __builtin_amdgcn_sched_barrier(0);                       // (the stores stay behind the loads)
+            if (col < a.vdim) store_rows(op + static_cast<size_t>(t) * o_stride, o_stride, col, row, a.L - t, O + O1);
+        };
+        walk_chunks<AHEAD>(a.chunks, step);
+    }
 }
 
 // ---- matrix memory, per chunk ------------------------------------------------------------------------------------------------------
@@ -442,8 +571,8 @@ __global__ __launch_bounds__(256) void memory_chunk_kernel(ChunkArgs a) {
         const int t = lane & 31;
         const bool in = t0 + t >= first && t0 + t < a.L;
         const size_t row = row0 + (t0 + t < a.L ? t0 + t : a.L - 1);
-        float f = in ? a.log_f[row * H + h] : 0.0f;
-        const float li = in ? a.log_i[row * H + h] : -1.0e30f;       // (a token that is not there: no weight, and its k is zero)
+        float f = in ? a.log_f[row * H + h] * kLog2e : 0.0f;
+        const float li = in ? a.log_i[row * H + h] * kLog2e : -1.0e30f;       // (a token that is not there: no weight, and its k is zero)
 #pragma unroll
         for (int d = 1; d < 32; d <<= 1) {
             const float o = __shfl_up(f, d, 32);
@@ -463,7 +592,7 @@ __global__ __launch_bounds__(256) void memory_chunk_kernel(ChunkArgs a) {
             I[t] = li;
             reinterpret_cast<float*>(out + Blk::f)[t] = f;
             reinterpret_cast<float*>(out + Blk::m)[t] = m;
-            reinterpret_cast<float*>(out + Blk::w)[t] = in ? expf(f_end - f + li - m_end) : 0.0f;
+            reinterpret_cast<float*>(out + Blk::w)[t] = in ? exp2_hw(f_end - f + li - m_end) : 0.0f;
         }
     }
     __syncthreads();
@@ -484,7 +613,7 @@ __global__ __launch_bounds__(256) void memory_chunk_kernel(ChunkArgs a) {
 #pragma unroll
         for (int i = 0; i < 4; i++) {
             const int t = rt * 16 + 4 * g + i, u = ct * 16 + r16;
-            Pm[t * kSqRow + u] = u <= t ? s[i] * expf(F[t] - F[u] + I[u] - M[t]) : 0.0f;
+            Pm[t * kSqRow + u] = u <= t ? s[i] * exp2_hw(F[t] - F[u] + I[u] - M[t]) : 0.0f;
         }
     }
     for (int u = tid; u < Blk::parts * 2 * KS * 64; u += 256) {      // q
@@ -508,110 +637,164 @@ __global__ __launch_bounds__(256) void memory_chunk_kernel(ChunkArgs a) {
     if (wv == 0) store_square(Pm, nullptr, out + Blk::p, lane);
 }
 
-// grid (column blocks of 16, the normalizer's column included, heads, sequences), one wavefront
+// grid (heads, column blocks of 16 with the normalizer's column, sequences), four wavefronts as above, the read-out a chunk behind
+// (one barrier per chunk, two buffers).  Logarithms to base 2 throughout.
 template <typename T, int DP>
-__global__ __launch_bounds__(kWave, 1) void memory_walk_kernel(ChunkArgs a) {
+__global__ __launch_bounds__(4 * kWave, 1) void memory_walk_kernel(ChunkArgs a) {
     constexpr bool SPLIT = __is_same(T, F16);
     using Blk = MemoryBlock<DP, SPLIT>;
-    constexpr int KS = DP / 32, NT = DP / 16, PT = Blk::parts;
-    const int lane = threadIdx.x, r16 = lane & 15, g = lane >> 4, h = blockIdx.y, b = blockIdx.z, H = a.H, columns = a.vdim + 1;
-    const int col = blockIdx.x * 16 + r16;
+    constexpr int KS = DP / 32, KH = KS / 2, NH = DP / 32, PT = Blk::parts, AHEAD = walk_ahead(DP);
+    __shared__ u32x4_a sh_s[2][2][KS][kWave], sh_v[2][PT][kWave];    // [buffer][part]
+    __shared__ float sh_m[2];
+    const int lane = threadIdx.x & 63, wv = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), r16 = lane & 15, g = lane >> 4;
+    const int h = blockIdx.x, b = blockIdx.z, H = a.H, columns = a.vdim + 1, col = blockIdx.y * 16 + r16;
     const bool value = col < a.vdim, norm = col == a.vdim;
     const size_t row0 = static_cast<size_t>(b) * a.L, head = static_cast<size_t>(b) * H + h;
-    const char* base = a.workspace + head * a.chunks * Blk::size + lane * 16;
-    float* sp = a.state + (head * columns + (col < columns ? col : 0)) * a.dim;
-    float* mp = a.m + head * gridDim.x + blockIdx.x;
-    floatx4_a S[NT];
-    load_state<NT>(sp, a.dim, g, S);
-    float m = *mp;
-
-    u32x4_a qi[PT][2][KS], ko[PT][NT], pm[2][2];
-    floatx4_a F[2], M[2], W[2];
-    float f_end, m_loc, v[2][4];
-    auto at = [&](const char* blk, int off) { return *reinterpret_cast<const u32x4_a*>(blk + off); };
-    auto load_qi = [&](const char* blk) {
-        static_for<PT * 2 * KS>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-            qi[i / (2 * KS)][i / KS % 2][i % KS] = at(blk, Blk::q_in + i * 1024);
+    const char* base = a.workspace + head * a.chunks * Blk::size;
+    const uint32_t lane16 = lane * 16, g16 = g * 16;
+    auto at = [&](const char* blk, int off) { return *reinterpret_cast<const u32x4_a*>(blk + off + lane16); };
+    auto scalars = [&](const char* blk, int off) { return *reinterpret_cast<const floatx4_a*>(blk + off + g16); };
+    if (wv < 2) {
+        const int c0 = wv * (DP / 2);
+        float* sp = a.state + (head * columns + (col < columns ? col : 0)) * a.dim + c0;
+        float* mp = a.m + head * gridDim.y + blockIdx.y;
+        floatx4_a S[NH], W[AHEAD][2];
+        load_state<NH>(sp, a.dim - c0, g, S);
+        float m = *mp * kLog2e, f_end[AHEAD], m_loc[AHEAD];
+        u32x4_a ko[AHEAD][PT][NH];
+        Rows<T> v[AHEAD][2];
+        auto load_ko = [&](auto P, const char* blk) {
+            constexpr int p = decltype(P)::value;
+            static_for<PT * NH>([&](auto J) {
+                constexpr int j = decltype(J)::value, part = j / NH, i = j % NH;
+                ko[p][part][i] = at(blk + wv * NH * 1024, Blk::k_out + part * Blk::kMat + i * 1024);
+            });
+        };
+        auto load_rest = [&](auto P, const char* blk, int t) {
+            constexpr int p = decltype(P)::value;
+            v[p][0].load(t);
+            v[p][1].load(t);
+            W[p][0] = scalars(blk, Blk::w);
+            W[p][1] = scalars(blk, Blk::w + 64);
+            f_end[p] = *reinterpret_cast<const float*>(blk + Blk::f + 31 * 4);
+            m_loc[p] = *reinterpret_cast<const float*>(blk + Blk::m + 31 * 4);
+        };
+        static_for<AHEAD>([&](auto P) {
+            constexpr int p = decltype(P)::value;
+            const int n = p < a.chunks ? p : a.chunks - 1;
+            const char* blk = base + static_cast<size_t>(n) * Blk::size;
+            v[p][0] = rows_of<T>(a, row0, h, value ? col : 0, 4 * g);
+            v[p][1] = rows_of<T>(a, row0, h, value ? col : 0, 16 + 4 * g);
+            load_rest(P, blk, a.t0 + n * kChunk);
+            load_ko(P, blk);
         });
-    };
-    auto load_ko = [&](const char* blk) {
-        static_for<PT * NT>([&](auto J) { constexpr int j = decltype(J)::value; ko[j / NT][j % NT] = at(blk, Blk::k_out + j * 1024); });
-    };
-    auto load_rest = [&](const char* blk, int t) {
-        static_for<2>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-            pm[0][i] = at(blk, Blk::p + i * 1024);
-            pm[1][i] = at(blk, Blk::p + Blk::kSq + i * 1024);
-            const char* sc = blk - lane * 16 + (i * 16 + 4 * g) * 4;
-            F[i] = *reinterpret_cast<const floatx4_a*>(sc + Blk::f);
-            M[i] = *reinterpret_cast<const floatx4_a*>(sc + Blk::m);
-            W[i] = *reinterpret_cast<const floatx4_a*>(sc + Blk::w);
-        });
-        f_end = *reinterpret_cast<const float*>(blk - lane * 16 + Blk::f + 31 * 4);
-        m_loc = *reinterpret_cast<const float*>(blk - lane * 16 + Blk::m + 31 * 4);
-#pragma unroll
-        for (int rt = 0; rt < 2; rt++)
-#pragma unroll
-            for (int i = 0; i < 4; i++) {
-                const float x = value_at<T>(a, row0, t + rt * 16 + 4 * g + i, h, value ? col : 0);
-                v[rt][i] = value ? x : 1.0f;
-            }
-    };
-    load_qi(base);
-    load_rest(base, a.t0);
-    load_ko(base);
-    for (int n = 0; n < a.chunks; n++) {
-        const int t = a.t0 + n * kChunk, next = n + 1 < a.chunks ? n + 1 : n;
-        const char* blk = base + static_cast<size_t>(next) * Blk::size;
-        u32x4_a sh[KS], sl[KS];
-        static_for<KS>([&](auto I) { constexpr int i = decltype(I)::value; split_tiles(S[2 * i], S[2 * i + 1], sh[i], sl[i]); });
-        floatx4_a O[2], O1[2], Pv[2];
-#pragma unroll
-        for (int rt = 0; rt < 2; rt++) O[rt] = O1[rt] = Pv[rt] = floatx4_a{0, 0, 0, 0};
-        static_for<KS>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-#pragma unroll
-            for (int rt = 0; rt < 2; rt++) {
-                O[rt] = mm(qi[0][rt][i], sh[i], O[rt]);
-                O1[rt] = mm(qi[0][rt][i], sl[i], O1[rt]);
-                if constexpr (SPLIT) O1[rt] = mm(qi[PT - 1][rt][i], sh[i], O1[rt]);
-            }
-        });
-        load_qi(blk);
-        const floatx4_a V[2] = {floatx4_a{v[0][0], v[0][1], v[0][2], v[0][3]}, floatx4_a{v[1][0], v[1][1], v[1][2], v[1][3]}};
-        u32x4_a vh, vl, xh, xl;
-        split_tiles(V[0], V[1], vh, vl);
-#pragma unroll
-        for (int rt = 0; rt < 2; rt++) {
-            Pv[rt] = mm(pm[0][rt], vh, Pv[rt]);
-            Pv[rt] = mm(pm[1][rt], vh, Pv[rt]);
-            if constexpr (SPLIT) Pv[rt] = mm(pm[0][rt], vl, Pv[rt]);
-        }
-        const float m_end = fmaxf(f_end + m, m_loc), keep = expf(f_end + m - m_end), take = expf(m_loc - m_end);
-        split_tiles(V[0] * W[0] * take, V[1] * W[1] * take, xh, xl);
-        static_for<NT>([&](auto J) { constexpr int j = decltype(J)::value; S[j] *= keep; });
-        static_for<NT>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[0][j], xh, S[j]); });
-        static_for<NT>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[0][j], xl, S[j]); });
-        if constexpr (SPLIT) static_for<NT>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[PT - 1][j], xh, S[j]); });
-        load_ko(blk);
-#pragma unroll
-        for (int rt = 0; rt < 2; rt++)
-#pragma unroll
-            for (int i = 0; i < 4; i++) {
-                const int tt = t + rt * 16 + 4 * g + i;
-                const float mt = fmaxf(F[rt][i] + m, M[rt][i]);
-                const float o = (expf(F[rt][i] + m - mt) * (O[rt][i] + O1[rt][i]) + expf(M[rt][i] - mt) * Pv[rt][i]) * a.q_scale;
-                if (tt < a.L) {
-                    if (value) a.o[((row0 + tt) * H + h) * a.vdim + col] = o;
-                    if (norm) a.den[(row0 + tt) * H + h] = fmaxf(fabsf(o), expf(-mt)) + 1e-6f;
+        auto step = [&](auto P, int n) {
+            constexpr int p = decltype(P)::value;
+            const int buf = n & 1, next = n + AHEAD < a.chunks ? n + AHEAD : a.chunks - 1;
+            const char* blk = base + static_cast<size_t>(next) * Blk::size;
+            floatx4_a V[2] = {v[p][0].get(), v[p][1].get()};
+            if (!value) V[0] = V[1] = floatx4_a{1, 1, 1, 1};
+            const float m_end = fmaxf(f_end[p] + m, m_loc[p]), keep = exp2_hw(f_end[p] + m - m_end), take = exp2_hw(m_loc[p] - m_end);
+            u32x4_a xh, xl;
+            if (wv == 0) {
+                if constexpr (SPLIT) {
+                    split_tiles(V[0], V[1], xh, xl);
+                    sh_v[buf][0][lane] = xh;
+                    sh_v[buf][PT - 1][lane] = xl;
+                } else {
+                    sh_v[buf][0][lane] = u32x4_a{pack_bf16(V[0][0], V[0][1]), pack_bf16(V[0][2], V[0][3]), pack_bf16(V[1][0], V[1][1]), pack_bf16(V[1][2], V[1][3])};
                 }
+                if (lane == 0) sh_m[buf] = m;
             }
-        m = m_end;
-        load_rest(blk, a.t0 + next * kChunk);
+            split_tiles(V[0] * W[p][0] * take, V[1] * W[p][1] * take, xh, xl);
+            __builtin_amdgcn_sched_barrier(0);
+            load_rest(P, blk, a.t0 + next * kChunk);
+            __builtin_amdgcn_sched_barrier(0);
+            static_for<KH>([&](auto I) {
+                constexpr int i = decltype(I)::value;
+                u32x4_a hi, lo;
+                split_tiles(S[2 * i], S[2 * i + 1], hi, lo);
+                sh_s[buf][0][wv * KH + i][lane] = hi;
+                sh_s[buf][1][wv * KH + i][lane] = lo;
+                S[2 * i] *= keep;
+                S[2 * i + 1] *= keep;
+            });
+            static_for<NH>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[p][0][j], xh, S[j]); });
+            static_for<NH>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[p][0][j], xl, S[j]); });
+            if constexpr (SPLIT) static_for<NH>([&](auto J) { constexpr int j = decltype(J)::value; S[j] = mm(ko[p][PT - 1][j], xh, S[j]); });
+            __builtin_amdgcn_sched_barrier(0);
+            load_ko(P, blk);
+            __builtin_amdgcn_sched_barrier(0);
+            m = m_end;
+            walk_barrier();
+        };
+        walk_chunks<AHEAD>(a.chunks, step);
+        if (col < columns) store_state<NH>(sp, a.dim - c0, g, S);
+        __syncthreads();                                             // (both halves have read the maximum long since)
+        if (threadIdx.x == 0) *mp = m / kLog2e;
+    } else {
+        const int rt = wv - 2, row = rt * 16 + 4 * g;
+        float* op = a.o + (row0 * H + h) * a.vdim;
+        float* np = a.den + row0 * H + h;
+        const uint32_t o_stride = static_cast<uint32_t>(H) * a.vdim;
+        u32x4_a qi[AHEAD][PT][KS], pm[AHEAD][2];
+        floatx4_a F[AHEAD], M[AHEAD];
+        auto load = [&](auto P, const char* blk) {
+            constexpr int p = decltype(P)::value;
+            static_for<PT * KS>([&](auto I) {
+                constexpr int i = decltype(I)::value, part = i / KS, k = i % KS;
+                qi[p][part][k] = at(blk + rt * KS * 1024, Blk::q_in + part * Blk::kMat + k * 1024);
+            });
+            pm[p][0] = at(blk + rt * 1024, Blk::p);
+            pm[p][1] = at(blk + rt * 1024, Blk::p + Blk::kSq);
+            F[p] = scalars(blk + rt * 64, Blk::f);
+            M[p] = scalars(blk + rt * 64, Blk::m);
+        };
+        static_for<AHEAD>([&](auto P) { load(P, base + static_cast<size_t>(P < a.chunks ? static_cast<int>(P) : a.chunks - 1) * Blk::size); });
+        LineFetch lines = line_fetch(base, Blk::size, a, lane);
+        lines.go(0);
+        auto step = [&](auto P, int n) {
+            constexpr int p = decltype(P)::value;
+            const int buf = n & 1, t = a.t0 + n * kChunk, next = n + AHEAD < a.chunks ? n + AHEAD : a.chunks - 1;
+            walk_barrier();
+            const float m = sh_m[buf];
+            const u32x4_a vh = sh_v[buf][0][lane];
+            floatx4_a O = {0, 0, 0, 0}, O1 = {0, 0, 0, 0}, Pv = {0, 0, 0, 0};
+            static_for<KS>([&](auto I) {
+                constexpr int i = decltype(I)::value;
+                const u32x4_a hi = sh_s[buf][0][i][lane], lo = sh_s[buf][1][i][lane];
+                O = mm(qi[p][0][i], hi, O);
+                O1 = mm(qi[p][0][i], lo, O1);
+                if constexpr (SPLIT) O1 = mm(qi[p][PT - 1][i], hi, O1);
+            });
+            Pv = mm(pm[p][0], vh, Pv);
+            Pv = mm(pm[p][1], vh, Pv);
+            if constexpr (SPLIT) Pv = mm(pm[p][0], sh_v[buf][PT - 1][lane], Pv);
+            // m_t is the larger of F_t + m and M_t: one of the two weights is 1
+            floatx4_a x, mt;
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const float old = F[p][i] + m, d = old - M[p][i], e = exp2_hw(-fabsf(d));
+                x[i] = ((d >= 0.0f ? 1.0f : e) * (O[i] + O1[i]) + (d >= 0.0f ? e : 1.0f) * Pv[i]) * a.q_scale;
+                mt[i] = fmaxf(old, M[p][i]);
+            }
+            __builtin_amdgcn_sched_barrier(0);
+            load(P, base + static_cast<size_t>(next) * Blk::size);
+            if (rt == 0) {
+                lines.drop();
+                lines.go(n + 1);
+            }
+            __builtin_amdgcn_sched_barrier(0);                       // (the stores stay behind the loads)
+            if (value) store_rows(op + static_cast<size_t>(t) * o_stride, o_stride, col, row, a.L - t, x);
+            if (norm) {
+#pragma unroll
+                for (int i = 0; i < 4; i++) x[i] = fmaxf(fabsf(x[i]), exp2_hw(-mt[i])) + 1e-6f;
+                store_rows(np + static_cast<size_t>(t) * H, H, 0, row, a.L - t, x);
+            }
+        };
+        walk_chunks<AHEAD>(a.chunks, step);
+        __syncthreads();
     }
-    if (col < columns) store_state<NT>(sp, a.dim, g, S);
-    if (lane == 0) *mp = m;
 }
 
 // ---- launchers -----------------------------------------------------------------------------------------------------------------------
@@ -638,7 +821,7 @@ static int delta_segment(const ChunkArgs& a, hipStream_t st) {
     if (int e = with_lds(&delta_chunk_kernel<T, DP>, lds)) return e;
     hipLaunchKernelGGL((delta_chunk_kernel<T, DP>), dim3(a.chunks, a.H, a.B), dim3(2 * DP), lds, st, a);
     if (int e = static_cast<int>(hipGetLastError())) return e;
-    hipLaunchKernelGGL((delta_walk_kernel<T, DP>), dim3((a.vdim + 15) / 16, a.H, a.B), dim3(kWave), 0, st, a);
+    hipLaunchKernelGGL((delta_walk_kernel<T, DP>), dim3(a.H, (a.vdim + 15) / 16, a.B), dim3(4 * kWave), 0, st, a);
     return static_cast<int>(hipGetLastError());
 }
 
@@ -650,7 +833,7 @@ static int memory_segment(const ChunkArgs& a, hipStream_t st) {
     if (int e = with_lds(&memory_chunk_kernel<T, DP>, lds)) return e;
     hipLaunchKernelGGL((memory_chunk_kernel<T, DP>), dim3(a.chunks, a.H, a.B), dim3(256), lds, st, a);
     if (int e = static_cast<int>(hipGetLastError())) return e;
-    hipLaunchKernelGGL((memory_walk_kernel<T, DP>), dim3(a.vdim / 16 + 1, a.H, a.B), dim3(kWave), 0, st, a);
+    hipLaunchKernelGGL((memory_walk_kernel<T, DP>), dim3(a.H, a.vdim / 16 + 1, a.B), dim3(4 * kWave), 0, st, a);
     return static_cast<int>(hipGetLastError());
 }
 
@@ -663,6 +846,11 @@ static int launch_chunks(const ChunkArgs& args, size_t workspace_bytes, int dtyp
     size_t fit = workspace_bytes / per;
     if (fit < 1) return static_cast<int>(hipErrorInvalidValue);
     const int step = fit < static_cast<size_t>(total) ? static_cast<int>(fit) : total;
+    // lines of up to eight chunks ahead, while those of an XCD's heads take half its 4 MB of L2; with more heads than that there
+    // are wavefronts enough to wait in turn
+    const size_t live = per * ((a.B * a.H + 7) / 8) / (static_cast<size_t>(a.B) * a.H);
+    const size_t ahead = (size_t{2} << 20) / live;
+    a.prefetch = ahead < 3 ? 0 : ahead > 8 ? 8 : static_cast<int>(ahead);
     for (int n = 0; n < total; n += step) {
         a.t0 = n * kChunk;
         a.chunks = n + step < total ? step : total - n;

@@ -109,6 +109,7 @@ constexpr int kRecurrentChunk = 32;
 struct ChunkArgs : ScanArgs {
     char* workspace;             // [B, H, chunks] blocks of chunk_block_bytes
     int t0, chunks;              // the segment: its first token in the call, how many chunks
+    int prefetch;                // chunks ahead of the walk whose lines are fetched into L2 (set by the launcher)
 };
 size_t chunk_block_bytes(bool delta, int dim, int dtype);
 int launch_delta_chunks(const ChunkArgs& a, size_t workspace_bytes, int dtype, hipStream_t st);
