@@ -327,7 +327,7 @@ __device__ __forceinline__ void walk_barrier() {
     asm volatile("" ::: "memory");
 }
 // chunks whose operands are in flight ahead of the one worked on, each in registers of its own
-constexpr int walk_ahead(int dp) { return dp <= 128 ? 2 : 1; }
+constexpr int walk_ahead(int dp) { return 1; }
 template <int AHEAD, typename F> __device__ __forceinline__ void walk_chunks(int chunks, F&& step) {
     for (int n = 0; n < chunks; n += AHEAD)
         static_for<AHEAD>([&](auto P) {
@@ -369,6 +369,7 @@ __global__ __launch_bounds__(4 * kWave, 1) void delta_walk_kernel(ChunkArgs a) {
     const uint32_t lane16 = lane * 16, g16 = g * 16;
     auto at = [&](const char* blk, int off) { return *reinterpret_cast<const u32x4_a*>(blk + off + lane16); };
     if (wv < 2) {
+        __builtin_amdgcn_s_setprio(3);                               // (ahead of another segment's chunks on the same compute unit)
         const int c0 = wv * (DP / 2);                                // this wavefront's first channel
         float* sp = a.state + ((static_cast<size_t>(b) * H + h) * a.vdim + cc) * a.dim + c0;
         floatx4_a S[NH], dec[AHEAD][NH];
@@ -655,6 +656,7 @@ __global__ __launch_bounds__(4 * kWave, 1) void memory_walk_kernel(ChunkArgs a) 
     auto at = [&](const char* blk, int off) { return *reinterpret_cast<const u32x4_a*>(blk + off + lane16); };
     auto scalars = [&](const char* blk, int off) { return *reinterpret_cast<const floatx4_a*>(blk + off + g16); };
     if (wv < 2) {
+        __builtin_amdgcn_s_setprio(3);
         const int c0 = wv * (DP / 2);
         float* sp = a.state + (head * columns + (col < columns ? col : 0)) * a.dim + c0;
         float* mp = a.m + head * gridDim.y + blockIdx.y;
@@ -798,6 +800,7 @@ __global__ __launch_bounds__(4 * kWave, 1) void memory_walk_kernel(ChunkArgs a) 
 }
 
 // ---- launchers -----------------------------------------------------------------------------------------------------------------------
+constexpr int kOverlapChunks = 64;        // chunks of a segment from which on a second stream is worth its events
 static int padded_dim(int dim) { return dim <= 64 ? 64 : dim <= 128 ? 128 : 256; }
 
 size_t chunk_block_bytes(bool delta, int dim, int dtype) {
@@ -813,55 +816,122 @@ static int with_lds(K kernel, size_t bytes) {
     return static_cast<int>(hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(bytes)));
 }
 
+// one segment: its chunks' operands, or the walk over them
 template <typename T, int DP>
-static int delta_segment(const ChunkArgs& a, hipStream_t st) {
+static int delta_launch(const ChunkArgs& a, bool walk, hipStream_t st) {
     static_assert(DeltaBlock<DP>::size % 16 == 0, "16-byte operands");
     constexpr size_t lds = 6 * static_cast<size_t>(kChunk) * (DP + 8) * 2 + (3 * kChunk * kSqRow + 2 * DP + kChunk) * sizeof(float);
     static_assert(lds <= 160 * 1024 && 6 * (DP + 8) * 2 >= 3 * DP * 4, "LDS");
-    if (int e = with_lds(&delta_chunk_kernel<T, DP>, lds)) return e;
-    hipLaunchKernelGGL((delta_chunk_kernel<T, DP>), dim3(a.chunks, a.H, a.B), dim3(2 * DP), lds, st, a);
-    if (int e = static_cast<int>(hipGetLastError())) return e;
-    hipLaunchKernelGGL((delta_walk_kernel<T, DP>), dim3(a.H, (a.vdim + 15) / 16, a.B), dim3(4 * kWave), 0, st, a);
+    if (walk) {
+        hipLaunchKernelGGL((delta_walk_kernel<T, DP>), dim3(a.H, (a.vdim + 15) / 16, a.B), dim3(4 * kWave), 0, st, a);
+    } else {
+        if (int e = with_lds(&delta_chunk_kernel<T, DP>, lds)) return e;
+        hipLaunchKernelGGL((delta_chunk_kernel<T, DP>), dim3(a.chunks, a.H, a.B), dim3(2 * DP), lds, st, a);
+    }
     return static_cast<int>(hipGetLastError());
 }
 
 template <typename T, int DP>
-static int memory_segment(const ChunkArgs& a, hipStream_t st) {
+static int memory_launch(const ChunkArgs& a, bool walk, hipStream_t st) {
     constexpr bool SPLIT = __is_same(T, F16);
     static_assert(MemoryBlock<DP, SPLIT>::size % 16 == 0, "16-byte operands");
     constexpr size_t lds = (SPLIT ? 4 : 2) * static_cast<size_t>(kChunk) * (DP + 8) * 2 + (kChunk * kSqRow + 3 * kChunk) * sizeof(float);
-    if (int e = with_lds(&memory_chunk_kernel<T, DP>, lds)) return e;
-    hipLaunchKernelGGL((memory_chunk_kernel<T, DP>), dim3(a.chunks, a.H, a.B), dim3(256), lds, st, a);
-    if (int e = static_cast<int>(hipGetLastError())) return e;
-    hipLaunchKernelGGL((memory_walk_kernel<T, DP>), dim3(a.H, a.vdim / 16 + 1, a.B), dim3(4 * kWave), 0, st, a);
+    if (walk) {
+        hipLaunchKernelGGL((memory_walk_kernel<T, DP>), dim3(a.H, a.vdim / 16 + 1, a.B), dim3(4 * kWave), 0, st, a);
+    } else {
+        if (int e = with_lds(&memory_chunk_kernel<T, DP>, lds)) return e;
+        hipLaunchKernelGGL((memory_chunk_kernel<T, DP>), dim3(a.chunks, a.H, a.B), dim3(256), lds, st, a);
+    }
     return static_cast<int>(hipGetLastError());
 }
 
-// The call's chunks in segments that the workspace holds.
+template <bool DELTA>
+static int launch_part(const ChunkArgs& a, bool walk, int dtype, hipStream_t st) {
+#define PQ_SEG(T, DP) (DELTA ? delta_launch<T, DP>(a, walk, st) : memory_launch<T, DP>(a, walk, st))
+#define PQ_SEG_D(T) (padded_dim(a.dim) == 64 ? PQ_SEG(T, 64) : padded_dim(a.dim) == 128 ? PQ_SEG(T, 128) : PQ_SEG(T, 256))
+    return dtype == 0 ? PQ_SEG_D(F16) : PQ_SEG_D(BF16);
+#undef PQ_SEG_D
+#undef PQ_SEG
+}
+
+// A stream beside the caller's, and events to order the two, for each host thread and device (default priority; kept for the
+// process).
+struct Side {
+    hipStream_t stream = nullptr;
+    hipEvent_t begin = nullptr, made[2] = {}, used[2] = {};
+    int ready = -1;              // -1: not tried, 0: there, otherwise the error
+};
+static Side& side_of_device() {
+    constexpr int kDevices = 16;
+    thread_local Side sides[kDevices];
+    int dev = 0;
+    if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= kDevices) dev = 0;
+    Side& s = sides[dev];
+    if (s.ready == -1) {
+        hipError_t e = hipStreamCreateWithFlags(&s.stream, hipStreamNonBlocking);
+        hipEvent_t* events[5] = {&s.begin, &s.made[0], &s.made[1], &s.used[0], &s.used[1]};
+        for (hipEvent_t* ev : events)
+            if (e == hipSuccess) e = hipEventCreateWithFlags(ev, hipEventDisableTiming);
+        s.ready = static_cast<int>(e);
+    }
+    return s;
+}
+
+// The call's chunks in segments that half the workspace holds; the next segment's operands are made, on a stream of their own,
+// while a segment is walked (a walk has few wavefronts).  One segment when the whole workspace holds the call.
 template <bool DELTA>
 static int launch_chunks(const ChunkArgs& args, size_t workspace_bytes, int dtype, hipStream_t st) {
     ChunkArgs a = args;
     const int total = (a.L + kChunk - 1) / kChunk;
     const size_t per = chunk_block_bytes(DELTA, a.dim, dtype) * a.B * a.H;
-    size_t fit = workspace_bytes / per;
+    const size_t fit = workspace_bytes / per;
     if (fit < 1) return static_cast<int>(hipErrorInvalidValue);
-    const int step = fit < static_cast<size_t>(total) ? static_cast<int>(fit) : total;
     // lines of up to eight chunks ahead, while those of an XCD's heads take half its 4 MB of L2; with more heads than that there
     // are wavefronts enough to wait in turn
     const size_t live = per * ((a.B * a.H + 7) / 8) / (static_cast<size_t>(a.B) * a.H);
     const size_t ahead = (size_t{2} << 20) / live;
     a.prefetch = ahead < 3 ? 0 : ahead > 8 ? 8 : static_cast<int>(ahead);
-    for (int n = 0; n < total; n += step) {
+    auto segment = [&](int n, int count) {
         a.t0 = n * kChunk;
-        a.chunks = n + step < total ? step : total - n;
-        int e;
-#define PQ_SEG(T, DP) (DELTA ? delta_segment<T, DP>(a, st) : memory_segment<T, DP>(a, st))
-#define PQ_SEG_D(T) (padded_dim(a.dim) == 64 ? PQ_SEG(T, 64) : padded_dim(a.dim) == 128 ? PQ_SEG(T, 128) : PQ_SEG(T, 256))
-        e = dtype == 0 ? PQ_SEG_D(F16) : PQ_SEG_D(BF16);
-#undef PQ_SEG_D
-#undef PQ_SEG
-        if (e) return e;
+        a.chunks = n + count < total ? count : total - n;
+    };
+    // few chunks, or no room for two segments: one after the other
+    const bool whole = fit >= static_cast<size_t>(total);
+    if ((whole && total < 2 * kOverlapChunks) || fit < 2) {
+        const int step = whole ? total : static_cast<int>(fit);
+        for (int n = 0; n < total; n += step) {
+            segment(n, step);
+            if (int e = launch_part<DELTA>(a, false, dtype, st)) return e;
+            if (int e = launch_part<DELTA>(a, true, dtype, st)) return e;
+        }
+        return 0;
     }
+    Side& side = side_of_device();
+    if (side.ready != 0) return side.ready;
+    // segments of a quarter of a call that fits, or of half the workspace
+    const int step = whole ? (total + 3) / 4 : static_cast<int>(fit / 2);
+    char* const half[2] = {a.workspace, a.workspace + step * per};
+#define PQ_TRY(call) do { const int e_ = static_cast<int>(call); if (e_) return e_; } while (0)
+    PQ_TRY(hipEventRecord(side.begin, st));
+    PQ_TRY(hipStreamWaitEvent(side.stream, side.begin, 0));
+    segment(0, step);
+    PQ_TRY(launch_part<DELTA>(a, false, dtype, st));
+    for (int n = 0, i = 0; n < total; n += step, i++) {
+        const int b = i & 1;
+        if (n + step < total) {
+            if (i > 0) PQ_TRY(hipStreamWaitEvent(side.stream, side.used[1 - b], 0));
+            segment(n + step, step);
+            a.workspace = half[1 - b];
+            PQ_TRY(launch_part<DELTA>(a, false, dtype, side.stream));
+            PQ_TRY(hipEventRecord(side.made[1 - b], side.stream));
+        }
+        if (i > 0) PQ_TRY(hipStreamWaitEvent(st, side.made[b], 0));
+        segment(n, step);
+        a.workspace = half[b];
+        PQ_TRY(launch_part<DELTA>(a, true, dtype, st));
+        PQ_TRY(hipEventRecord(side.used[b], st));
+    }
+#undef PQ_TRY
     return 0;
 }
 int launch_delta_chunks(const ChunkArgs& a, size_t workspace_bytes, int dtype, hipStream_t st) { return launch_chunks<true>(a, workspace_bytes, dtype, st); }

@@ -316,8 +316,8 @@ int launch_relu_sq(const void* x, void* y, size_t n, int dtype, hipStream_t st) 
 // ---- gelu (tanh form) times --------------------------------------------------------------------------------------------
 // 0.5 z (1 + tanh u) = z / (1 + exp(-2 u)), u = sqrt(2 / pi) (z + 0.044715 z^3)
 __device__ __forceinline__ float gelu_tanh(float z) {
-    const float u2 = 1.5957691216057308f * (z + 0.044715f * z * z * z);
-    return z / (1.0f + expf(-u2));
+    const float u2 = 1.5957691216057308f * __builtin_fmaf(0.044715f * z * z, z, z);
+    return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(u2 * -1.4426950408889634f));
 }
 
 // grid (column pieces, rows)

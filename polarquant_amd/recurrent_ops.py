@@ -16,8 +16,8 @@ from .layer_ops import _DTYPES, ConvState, _code, _ptr
 WINDOW_SMALL = 16          # new tokens per sequence up to which keys go to the ring before they are read
 MAX_DIM = 256              # of a recurrent head
 MAX_TAPS = 16
-CHUNKED_TOKENS = 64        # from this many tokens per sequence on, 16-bit recurrences run in chunks on the matrix cores
-WORKSPACE_BYTES = 160 << 20         # of a chunked recurrence, at most (what fits the last-level cache beside its other operands)
+CHUNKED_TOKENS = WINDOW_SMALL + 1     # from this many tokens per sequence on, 16-bit recurrences run in chunks on the matrix cores
+WORKSPACE_BYTES = 384 << 20         # of a chunked recurrence, at most
 
 
 class Step(NamedTuple):

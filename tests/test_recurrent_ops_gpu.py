@@ -303,3 +303,70 @@ def test_matrix_memory_recalls_a_far_token(gpu):
             assert err(memory_oracle(p[0], b, b, w, H, dim, vdim, cap, 1e-4)[1][-50:], want[-50:]) > 0.3
             for cuts in ([T], [440] + [1] * 60, cut(T, [100, 2])):
                 assert err(memory_run(gpu, q, b, b, w, H, dim, vdim, cap, 1e-4, cuts)[1], want[None]) < (2e-4 if dt == "f32" else 2.5 * TOL[dt]), (dt, far)
+
+
+# ---------------------------------------------------------------- chunked recurrences, longer calls
+@pytest.mark.parametrize("workspace", [1, 400_000, 3_000_000, 384 << 20])
+def test_chunks_in_segments(gpu, monkeypatch, workspace):
+    """Workspaces of one chunk, of a few, and of the whole call, whose segments are then made on a second stream while others
+    are walked; state handed from segment to segment and from call to call, the last chunk partial."""
+    monkeypatch.setattr(ops, "WORKSPACE_BYTES", workspace)
+    g = torch.Generator().manual_seed(11)
+    T = 4500
+    for cuts in ([T], [4200, 1, 299]):
+        t = delta_case(g, 1, T, 1, 2, 48, 20, 3, "bf16")
+        t["A_log"] -= 3.0                                        # (memories of hundreds of tokens)
+        want = delta_oracle(t, 0, 0, 1, 2, 48, 20, 1e-4)[0]
+        assert err(delta_run(gpu, t, cuts, 1, 2, 48, 20, 3, 1e-4)[0], want[None]) < TOL["bf16"], cuts
+        p = rand(g, 1, T, 2 * 32 + 2 * 20 + 2, dt="bf16")
+        p[:, :, -1] += 5.0
+        b, w = torch.zeros(1).bfloat16(), torch.ones(20).bfloat16()
+        want = memory_oracle(p[0], b, b, w, 1, 32, 20, 9.0, 1e-4)[1]
+        assert err(memory_run(gpu, p, b, b, w, 1, 32, 20, 9.0, 1e-4, cuts)[1], want[None]) < 2.5 * TOL["bf16"], cuts
+
+
+def test_chunks_agree_with_the_token_by_token_kernel(gpu, monkeypatch):
+    """A batch of many heads, whose results the plain implementation would take too long for."""
+    g = torch.Generator().manual_seed(12)
+    B, T, G, H, dim, vdim = 3, 700, 4, 8, 128, 128
+    t = delta_case(g, B, T, G, H, dim, vdim, 4, "bf16")
+    p = rand(g, B, T, 2 * H * 128 + 2 * H * 192 + 2 * H, dt="bf16")
+    p[:, :, -H:] += 4.0
+    b, w = torch.zeros(H).bfloat16(), torch.ones(H * 192).bfloat16()
+    start = torch.tensor([0, 333, 699], dtype=torch.int32, device=gpu)
+    runs = []
+    for tokens in (10 ** 9, 1):
+        monkeypatch.setattr(ops, "CHUNKED_TOKENS", tokens)
+        runs.append((delta_run(gpu, t, [T], G, H, dim, vdim, 4, 1e-4, start), memory_run(gpu, p, b, b, w, H, 128, 192, 12.0, 1e-4, [T], start)))
+    (d0, m0), (d1, m1) = runs
+    assert err(d1[0], d0[0].double()) < 1e-4 and err(d1[2], d0[2].double().cpu()) < 1e-4 and torch.equal(d1[3].rows, d0[3].rows)
+    first = start.tolist()
+    for i in range(B):
+        assert err(m1[1][i, first[i]:], m0[1][i, first[i]:].double()) < 1e-2
+
+
+def test_chunks_in_a_graph(gpu):
+    """Both streams of a long call captured; several replays with the program's own work between them, each from the same state."""
+    g = torch.Generator().manual_seed(13)
+    T, H, dim, vdim = 4200, 2, 64, 32
+    x = ops.DeltaInputs(*[rand(g, T, n, dt="bf16").to(gpu) for n in (H * dim, H * dim, H * vdim)], torch.full((T, H), 0.01, device=gpu),
+                        torch.full((T, H), 0.1, device=gpu), -rand(g, T, H * dim).abs().to(gpu) * 0.02, torch.rand(T, H, generator=g).to(gpu))
+    S = torch.zeros(1, H, vdim, dim, device=gpu)
+    step = Step(1, T, 0)
+    want = ops.delta_scan(x, S, step).clone()
+    end = S.clone()
+    side = torch.cuda.Stream()
+    side.wait_stream(torch.cuda.current_stream())
+    with torch.cuda.stream(side):
+        S.zero_()
+        ops.delta_scan(x, S, step)
+    torch.cuda.current_stream().wait_stream(side)
+    graph = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(graph):
+        got = ops.delta_scan(x, S, step)
+    for _ in range(4):
+        S.zero_()
+        graph.replay()
+        assert torch.equal(got, want) and torch.equal(S, end)
+        torch.cuda.synchronize()
+        _ = (got * 2).sum().item()
