@@ -177,6 +177,7 @@ int pq_memory_scan(const void* q, const void* k, const void* v, int64_t row_stri
     if (!q || !k || !v || !log_i || !log_f || !state || !m || !o || !den) return PQ_ERR_NULL_POINTER;
     if (int rc = check_scan(B, L, H, H, dim, vdim, dtype)) return rc;
     if (row_stride < static_cast<int64_t>(H) * (dim > vdim ? dim : vdim)) return PQ_ERR_BAD_STRIDE;
+    if (workspace && row_stride > (1 << 26)) return PQ_ERR_BAD_STRIDE;      // (a chunk's rows are addressed with 32 bits)
     if (workspace)
         if (int rc = check_chunks(false, B, H, dim, workspace, workspace_bytes, pos_dev, dtype)) return rc;
     pq::ChunkArgs a{};

@@ -327,7 +327,7 @@ __device__ __forceinline__ void walk_barrier() {
     asm volatile("" ::: "memory");
 }
 // chunks whose operands are in flight ahead of the one worked on, each in registers of its own
-constexpr int walk_ahead(int dp) { return 1; }
+constexpr int kWalkAhead = 1;
 template <int AHEAD, typename F> __device__ __forceinline__ void walk_chunks(int chunks, F&& step) {
     for (int n = 0; n < chunks; n += AHEAD)
         static_for<AHEAD>([&](auto P) {
@@ -359,7 +359,7 @@ __device__ __forceinline__ LineFetch line_fetch(const char* base, int block_byte
 template <typename T, int DP>
 __global__ __launch_bounds__(4 * kWave, 1) void delta_walk_kernel(ChunkArgs a) {
     using Blk = DeltaBlock<DP>;
-    constexpr int KS = DP / 32, KH = KS / 2, NH = DP / 32, AHEAD = walk_ahead(DP);
+    constexpr int KS = DP / 32, KH = KS / 2, NH = DP / 32, AHEAD = kWalkAhead;
     __shared__ u32x4_a sh_s[2][KS][kWave], sh_u[2][kWave];           // high and low parts
     __shared__ floatx4_a sh_r[2][2][kWave];                          // [half][row tile]
     const int lane = threadIdx.x & 63, wv = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), r16 = lane & 15, g = lane >> 4;
@@ -644,7 +644,7 @@ template <typename T, int DP>
 __global__ __launch_bounds__(4 * kWave, 1) void memory_walk_kernel(ChunkArgs a) {
     constexpr bool SPLIT = __is_same(T, F16);
     using Blk = MemoryBlock<DP, SPLIT>;
-    constexpr int KS = DP / 32, KH = KS / 2, NH = DP / 32, PT = Blk::parts, AHEAD = walk_ahead(DP);
+    constexpr int KS = DP / 32, KH = KS / 2, NH = DP / 32, PT = Blk::parts, AHEAD = kWalkAhead;
     __shared__ u32x4_a sh_s[2][2][KS][kWave], sh_v[2][PT][kWave];    // [buffer][part]
     __shared__ float sh_m[2];
     const int lane = threadIdx.x & 63, wv = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), r16 = lane & 15, g = lane >> 4;

@@ -46,7 +46,7 @@ ODD = config(70, 101, [parallel((3, 1, 20, 12, 7, 0.4), (3, 1, 7, 10, 7), 0.8, 0
 # ones: a window of the token itself, a filter of one tap, single heads, one pass over all layers
 ONES = config(96, 144, [memory(1, 32, 32, 10.0, 64), parallel((1, 1, 16, 16, 1, 1.0), (1, 1, 16, 16, 1), 1.0, 1.0, 32)], (0, 2, 1), logit_scale=1.0)
 # wide heads, no loop
-WIDE = config(256, 160, [parallel((2, 1, 136, 128, 130, 0.1), (2, 1, 128, 128, 4), 0.6, 0.9, 256), memory(1, 200, 136, 12.0, 128)])
+WIDE = config(256, 160, [parallel((2, 1, 136, 128, 130, 0.1), (2, 1, 128, 128, 4), 0.65, 0.85, 288), memory(1, 200, 136, 11.0, 128)])
 ALL = {"even": EVEN, "odd": ODD, "ones": ONES, "wide": WIDE}
 RANKS = {"even": (40, 16), "odd": (5, 11), "ones": (1, 3), "wide": (64, 32)}
 
