@@ -83,7 +83,7 @@ def test_every_mechanism_shows():
     they would notice it."""
     cfg = kc.changed(kc.EVEN, lambda c: (c.update(logit_softcap=2.0), [c["layers"][i]["mixer"]["left"].update(scale=1.0) for i in (0, 2)]))   # (sharp attention)
     w = kc.weights(cfg, 13, kc.RANKS["even"])
-    t = kc.tokens(70, cfg["vocab"], 6)
+    t = kc.tokens(46, cfg["vocab"], 6)
     want = ko.forward(t, cfg, w)
     off = lambda c=cfg, x=w: kc.rel_rms(ko.forward(t, c, x), want)
     left = lambda c, i: c["layers"][i]["mixer"]["left"]
